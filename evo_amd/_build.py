@@ -3,8 +3,10 @@
 The sources are grouped into components, one library each, so that a process builds and loads only what its model calls:
   core          dense layers, norms, embedding, scoring tail -- every model
   stripedhyena  the Hyena operator and the causal attention of the StripedHyena models
-  mixers        the mixers described by a config.json model (decayed linear attention, windowed latent attention) and the
-                token-local kernels around them
+  mixers        what every model described by a config.json shares: the token-local kernels around the mixers, softmax attention of prompts
+  lightning, latent, heads, rglru
+                one mechanism each: decayed linear attention, latent attention, attention with cached keys and values, gated linear
+                recurrence
 
 In-tree build: the .so files land in evo_amd/_lib/ so they travel with the repo snapshot to the GPU box
 (they are git-ignored).  hipcc cross-compiles without a GPU.
@@ -32,17 +34,21 @@ COMPONENTS = {
         "evo_linear_small_m_bf16", "evo_norm_linear_small_m_bf16", "evo_mlp_gate_small_m_bf16", "evo_norm_mlp_gate_small_m_bf16",
         "evo_hyena_decode_fused_small_m", "evo_linear_mfma_bf16", "evo_linear_mfma_nf_bf16", "evo_mlp_gate_mfma_bf16",
         "evo_mlp_gate_mfma_nf_bf16", "evo_linear_xblk_mfma_bf16", "evo_linear_xblk_mfma_nf_bf16", "evo_linear_t_mfma_bf16",
-        "evo_linear_t_mfma_nf_bf16", "evo_linear_silu_mfma_bf16", "evo_postnorm_linear_small_m_bf16",
+        "evo_linear_t_mfma_nf_bf16", "evo_linear_act_mfma_bf16", "evo_postnorm_linear_small_m_bf16",
         "evo_postnorm_mlp_gate_small_m_bf16", "evo_probe_copy_f4", "evo_probe_mfma_bf16",
     ]),
     "stripedhyena": ("_stripedhyena", ["attn", "attn_w64", "hyena", "hyena_ct"], ["attn_common.h"], [
         "evo_hyena_seg_state", "evo_hyena_carry_scan", "evo_hyena_carry_add", "evo_hyena_apply", "evo_hyena_step", "evo_hyena_ct",
         "evo_attn_fwd_causal_bf16", "evo_attn_decode_bf16",
     ]),
-    "mixers": ("_mixers", ["stream", "lightning", "latent"], ["mixers_common.h"], [
-        "evo_embed_stream", "evo_postnorm_residual", "evo_rmsnorm_stream", "evo_gated_norm", "evo_silu_gate", "evo_silu_cols", "evo_lightning_chunk_bf16",
-        "evo_lightning_recurrent", "evo_latent_prep", "evo_window_attn", "evo_latent_absorb", "evo_latent_decode", "evo_latent_up",
+    "mixers": ("_mixers", ["stream", "window_attn"], ["mixers_common.h"], [
+        "evo_embed_stream", "evo_postnorm_residual", "evo_sum_norm", "evo_rmsnorm_stream", "evo_gated_norm", "evo_silu_gate", "evo_act_cols",
+        "evo_window_attn",
     ]),
+    "lightning": ("_lightning", ["lightning"], ["mixers_common.h"], ["evo_lightning_chunk_bf16", "evo_lightning_recurrent"]),
+    "latent": ("_latent", ["latent"], ["mixers_common.h"], ["evo_latent_prep", "evo_latent_absorb", "evo_latent_decode", "evo_latent_up"]),
+    "heads": ("_heads", ["heads"], ["mixers_common.h"], ["evo_heads_prep", "evo_heads_decode", "evo_heads_merge"]),
+    "rglru": ("_rglru", ["rglru"], ["mixers_common.h"], ["evo_rglru_chunk_bf16", "evo_rglru_step_bf16", "evo_rglru_any"]),
 }
 
 # every symbol include/evo_mi355x.h declares

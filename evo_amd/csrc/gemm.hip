@@ -47,7 +47,7 @@ struct GemmArgs {
     const float* rs = nullptr;               // SCALE: 1 / (rms + eps) per token row, applied to the accumulators in the epilogue
     float* ss = nullptr;                     // STATS: partial sums of squares of the stored rows, [N / 128 strips][ss_ld] fp32
     int64_t ss_ld = 0;
-    int act_cols = 0;                        // ACT, mode 0: columns [0, act_cols) of the result go through SiLU (a multiple of 256)
+    int act_cols = 0;                        // ACT, mode 0: columns [0, act_cols) of the result go through the activation (a multiple of 256)
     int64_t w_rows = 0;                      // MODE 3 + SCALE: rows of the token matrix (the kernel's "W" operand): B T
     int tm_tiles = 0, row_skip = 0;          // MODE 3 + SCALE: a batch row = tm_tiles column tiles; its tokens start row_skip rows further per batch row
 };
@@ -377,7 +377,7 @@ static_assert(!GE_FULL || GE_ORDER == 1, "GE_FULL pairs the strips of GE_ORDER 1
 //     in modes 0 / 1 (eight values per lane and tile: one per m tile) and along the REGISTERS in mode 3 (the swapped launch: 32 values per
 //     lane, the eight columns of its four strips).  Mode 3 also reads its token rows from the residual stream itself: z^T position
 //     p = b Tm + t is row p + b row_skip of x (tail form of z^T: rows of Tm = T - row_skip positions, a tile never straddles two batch rows).
-template <bool BIAS, bool RES, int MODE, bool XB = false, int NF = 0, int ACT = 0>   // ACT: gate of mode 1 (act_gate2), SiLU of the first columns in mode 0; MODE 0: y [M, N]; 1: gated MLP, a [M, N / 2]; (2: retired with csrc/hyena_cs.hip in round 5);
+template <bool BIAS, bool RES, int MODE, bool XB = false, int NF = 0, int ACT = 0>   // ACT: gate of mode 1 (act_gate2), activation of the first columns in mode 0 (1 SiLU, 2 tanh-form GELU, 3 square of relu); MODE 0: y [M, N]; 1: gated MLP, a [M, N / 2]; (2: retired with csrc/hyena_cs.hip in round 5);
                                                             // 3: y [M, N] with the bias indexed by ROW (the swapped-operand launch: evo_linear_t_mfma_bf16)
 __global__ __launch_bounds__(256, 1) void gemmr_bf16_kernel(GemmArgs a) {
     constexpr bool STATS = (NF & 1) != 0, SCALE = (NF & 2) != 0;
@@ -783,7 +783,10 @@ __global__ __launch_bounds__(256, 1) void gemmr_bf16_kernel(GemmArgs a) {
                 asm volatile("s_waitcnt vmcnt(0)" : "+v"(rsq[0][0]), "+v"(rsq[0][1]), "+v"(rsq[1][0]), "+v"(rsq[1][1]), "+v"(rsq[2][0]),
                              "+v"(rsq[2][1]), "+v"(rsq[3][0]), "+v"(rsq[3][1]) :: "memory");
             }
-            const float act_k1 = n0 < a.act_cols ? -1.4426950408889634f : 0.f, act_k0 = n0 < a.act_cols ? 0.f : -1000.f;   // ACT: exponent of the logistic
+            // ACT: SiLU and tanh-form GELU are v * logistic(p(v)), the exponent of the logistic k0 + k1 v (+ k3 v^3); square of relu: max(v, k1) (k0 + k3 max(v, k1))
+            const bool act_on = n0 < a.act_cols;
+            const float act_k1 = ACT == 3 ? (act_on ? 0.f : -INFINITY) : (act_on ? (ACT == 2 ? -2.3022081981443250f : -1.4426950408889634f) : 0.f);
+            const float act_k0 = ACT == 3 ? (act_on ? 0.f : 1.f) : (act_on ? 0.f : -1000.f), act_k3 = ACT == 3 ? (act_on ? 1.f : 0.f) : (act_on ? -0.1029432395800235f : 0.f);
             float ssq = 0.f, sst[4];                             // STATS: the running sum of squares of this lane's row in m tile j; stored totals
             if (BIAS && MODE != 3) {                             // the lane's eight columns of every strip
 #pragma unroll
@@ -847,9 +850,14 @@ __global__ __launch_bounds__(256, 1) void gemmr_bf16_kernel(GemmArgs a) {
                     v[0] += bf_lo(r[0]); v[1] += bf_hi(r[0]); v[2] += bf_lo(r[1]); v[3] += bf_hi(r[1]);
                     v[4] += bf_lo(r[2]); v[5] += bf_hi(r[2]); v[6] += bf_lo(r[3]); v[7] += bf_hi(r[3]);
                 }
-                if constexpr (ACT == 1 && MODE == 0) {               // silu(v), or v * 1 in the tiles behind act_cols: no branch among the asm stores
+                if constexpr (ACT && MODE == 0) {                    // (v * 1 in the tiles behind act_cols: no branch among the asm stores)
 #pragma unroll
-                    for (int e = 0; e < 8; ++e) v[e] *= __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(fmaf(v[e], act_k1, act_k0)));
+                    for (int e = 0; e < 8; ++e) {
+                        if constexpr (ACT == 3) {
+                            const float m = fmaxf(v[e], act_k1);
+                            v[e] = m * fmaf(m, act_k3, act_k0);
+                        } else v[e] *= __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(fmaf(v[e], ACT == 2 ? fmaf(v[e] * v[e], act_k3, act_k1) : act_k1, act_k0)));
+                    }
                 }
                 // the one rounding
                 g_u32x4 o;
@@ -993,13 +1001,15 @@ extern "C" int evo_linear_mfma_nf_bf16(const void* x, const void* w, const void*
     return evo_launch_status();
 }
 
-// y [M, N] = x . w^T with SiLU on columns [0, act_cols): the input projection of a linear-attention mixer, whose q, k, v are activated and
-// whose gate is not.  act_cols % 256 == 0; N % 256 == 0, K % 64 == 0, K >= 128, operands below 4 GiB.
-extern "C" int evo_linear_silu_mfma_bf16(const void* x, const void* w, void* y, int64_t M, int64_t N, int64_t K, int64_t act_cols, void* stream) {
-    if (M <= 0 || N <= 0 || N % GBN != 0 || K % GBK != 0 || K < 2 * GBK || N > 0x7fffffff / 2 || act_cols < 0 || act_cols > N || act_cols % GBN != 0) return -1;
+// y [M, N] = act(x . w^T + bias) on columns [0, act_cols), without act behind them: input projections that activate some of their parts, and
+// ungated feed-forwards.  act 1: SiLU, 2: GELU (tanh form), 3: square of relu; act_cols % 256 == 0; N % 256 == 0, K % 64 == 0, K >= 128,
+// operands below 4 GiB.
+extern "C" int evo_linear_act_mfma_bf16(const void* x, const void* w, const void* bias, void* y, int64_t M, int64_t N, int64_t K, int64_t act_cols,
+                                        int64_t act, void* stream) {
+    if (M <= 0 || N <= 0 || N % GBN != 0 || K % GBK != 0 || K < 2 * GBK || N > 0x7fffffff / 2 || act_cols < 0 || act_cols > N || act_cols % GBN != 0 || act < 1 || act > 3) return -1;
     if (M * K * 2 >= 0xffffffffll || N * K * 2 >= 0xffffffffll) return -1;
     GemmArgs a;
-    a.x = (const unsigned char*)x; a.w = (const unsigned char*)w; a.bias = nullptr; a.res = nullptr; a.y = (uint16_t*)y;
+    a.x = (const unsigned char*)x; a.w = (const unsigned char*)w; a.bias = (const uint16_t*)bias; a.res = nullptr; a.y = (uint16_t*)y;
     a.M = M; a.N = (int)N; a.K = (int)K;
     a.act_cols = (int)act_cols;
     a.tiles_n = (int)(N / GBN);
@@ -1014,7 +1024,10 @@ extern "C" int evo_linear_silu_mfma_bf16(const void* x, const void* w, void* y, 
         n &= ~7;
         return n < 8 ? 8 : n;
     }();
-    hipLaunchKernelGGL((gemmr_bf16_kernel<false, false, 0, false, 0, 1>), dim3((unsigned)n_cu), dim3(256), 0, (hipStream_t)stream, a);
+#define EVO_ACT(BIAS, ACT) hipLaunchKernelGGL((gemmr_bf16_kernel<BIAS, false, 0, false, 0, ACT>), dim3((unsigned)n_cu), dim3(256), 0, (hipStream_t)stream, a)
+    if (bias) { if (act == 1) EVO_ACT(true, 1); else if (act == 2) EVO_ACT(true, 2); else EVO_ACT(true, 3); }
+    else { if (act == 1) EVO_ACT(false, 1); else if (act == 2) EVO_ACT(false, 2); else EVO_ACT(false, 3); }
+#undef EVO_ACT
     return evo_launch_status();
 }
 

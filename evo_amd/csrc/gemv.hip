@@ -630,12 +630,13 @@ __global__ __launch_bounds__(256) void gemv_gate_kernel(const uint4* __restrict_
 
 // ---- a sublayer's closing norm folded into the next one's first layer (decode form of models with an fp32 residual stream):
 //   x' = x + y / sqrt(mean(y^2) + eps) * (off + g)       (rows of the stream; workgroup 0 also stores them)
-//   plain: z = bf16(x') . W^T          gated: a = act(bf16(x') . W1^T) * (bf16(x') . W2^T), w = [W1; W2] or its grouped order
+//   SUM: x' = t / sqrt(mean(t^2) + eps) * (off + g), t = alpha x + y
+//   plain: z = bf16(x') . W^T (act 3: through the square of relu)         gated: a = act(bf16(x') . W1^T) * (bf16(x') . W2^T), w = [W1; W2] or its grouped order
 // Every workgroup rebuilds the M rows -- 8 bytes per element from L2 -- into LDS while its first weight requests are under way.
-template <int M, bool GATE>
+template <int M, bool GATE, bool SUM>
 __global__ __launch_bounds__(256) void postnorm_gemv_kernel(const uint4* __restrict__ y, const uint4* __restrict__ g, const float4* __restrict__ x,
                                                             float4* __restrict__ x_out, const uint4* __restrict__ w, uint16_t* __restrict__ out, int N,
-                                                            int nvec, float eps, float off, int grouped, int act) {
+                                                            int nvec, float alpha, float eps, float off, int grouped, int act) {
     extern __shared__ uint4 pn_x[];                              // [M][nvec]
     __shared__ float red[M][4];
     const int tid = threadIdx.x, lane = tid & 63;
@@ -659,7 +660,16 @@ __global__ __launch_bounds__(256) void postnorm_gemv_kernel(const uint4* __restr
 #pragma unroll
     for (int m = 0; m < M; ++m) {
         float ss = 0.f;
-        for (int v = tid; v < nvec; v += 256) ss = gv_sumsq8(y[(int64_t)m * nvec + v], ss);
+        for (int v = tid; v < nvec; v += 256) {
+            const uint4 yv = y[(int64_t)m * nvec + v];
+            if (SUM) {
+                const float4 a = x[((int64_t)m * nvec + v) * 2], b = x[((int64_t)m * nvec + v) * 2 + 1];
+                const float t[8] = {fmaf(alpha, a.x, bf_lo(yv.x)), fmaf(alpha, a.y, bf_hi(yv.x)), fmaf(alpha, a.z, bf_lo(yv.y)), fmaf(alpha, a.w, bf_hi(yv.y)),
+                                    fmaf(alpha, b.x, bf_lo(yv.z)), fmaf(alpha, b.y, bf_hi(yv.z)), fmaf(alpha, b.z, bf_lo(yv.w)), fmaf(alpha, b.w, bf_hi(yv.w))};
+#pragma unroll
+                for (int e = 0; e < 8; ++e) ss = fmaf(t[e], t[e], ss);
+            } else ss = gv_sumsq8(yv, ss);
+        }
         ss = wave_sum(ss);
         if (lane == 0) red[m][wave] = ss;
     }
@@ -670,10 +680,17 @@ __global__ __launch_bounds__(256) void postnorm_gemv_kernel(const uint4* __restr
         for (int v = tid; v < nvec; v += 256) {
             const uint4 yv = y[(int64_t)m * nvec + v], gv = g[v];
             float4 a = x[((int64_t)m * nvec + v) * 2], b = x[((int64_t)m * nvec + v) * 2 + 1];
+            if (SUM) {
+                a.x = fmaf(alpha, a.x, bf_lo(yv.x)) * inv * (off + bf_lo(gv.x)); a.y = fmaf(alpha, a.y, bf_hi(yv.x)) * inv * (off + bf_hi(gv.x));
+                a.z = fmaf(alpha, a.z, bf_lo(yv.y)) * inv * (off + bf_lo(gv.y)); a.w = fmaf(alpha, a.w, bf_hi(yv.y)) * inv * (off + bf_hi(gv.y));
+                b.x = fmaf(alpha, b.x, bf_lo(yv.z)) * inv * (off + bf_lo(gv.z)); b.y = fmaf(alpha, b.y, bf_hi(yv.z)) * inv * (off + bf_hi(gv.z));
+                b.z = fmaf(alpha, b.z, bf_lo(yv.w)) * inv * (off + bf_lo(gv.w)); b.w = fmaf(alpha, b.w, bf_hi(yv.w)) * inv * (off + bf_hi(gv.w));
+            } else {
             a.x += bf_lo(yv.x) * inv * (off + bf_lo(gv.x)); a.y += bf_hi(yv.x) * inv * (off + bf_hi(gv.x));
             a.z += bf_lo(yv.y) * inv * (off + bf_lo(gv.y)); a.w += bf_hi(yv.y) * inv * (off + bf_hi(gv.y));
             b.x += bf_lo(yv.z) * inv * (off + bf_lo(gv.z)); b.y += bf_hi(yv.z) * inv * (off + bf_hi(gv.z));
             b.z += bf_lo(yv.w) * inv * (off + bf_lo(gv.w)); b.w += bf_hi(yv.w) * inv * (off + bf_hi(gv.w));
+            }
             pn_x[m * nvec + v] = make_uint4(pack_bf2(a.x, a.y), pack_bf2(a.z, a.w), pack_bf2(b.x, b.y), pack_bf2(b.z, b.w));
             if (blockIdx.x == 0) {
                 x_out[((int64_t)m * nvec + v) * 2] = a;
@@ -733,38 +750,46 @@ __global__ __launch_bounds__(256) void postnorm_gemv_kernel(const uint4* __restr
             } else {
 #pragma unroll
                 for (int r = 0; r < 4; ++r)
-                    if (n0 + r < N) out[(int64_t)m * N + n0 + r] = f_to_bf(acc[r][m]);
+                    if (n0 + r < N) {
+                        const float z = act ? fmaxf(acc[r][m], 0.f) : acc[r][m];
+                        out[(int64_t)m * N + n0 + r] = f_to_bf(act ? z * z : z);
+                    }
             }
         }
     }
 }
 
 static int postnorm_gemv_launch(const void* y, const void* g, const float* x, float* x_out, const void* w, void* out, int64_t M, int64_t N, int64_t K,
-                                float eps, float off, bool gate, int64_t grouped, int64_t act, void* stream) {
+                                float alpha, bool sum, float eps, float off, bool gate, int64_t grouped, int64_t act, void* stream) {
     if (M < 1 || M > 4 || N <= 0 || N > 0x3fffffff || K <= 0 || K % 8 != 0 || K > 8192 || !y || !g || !x || !x_out || !w || !out || x == x_out) return -1;
-    if (gate && ((act != 0 && act != 1) || (grouped && N % 32 != 0))) return -1;
+    if (gate ? ((act != 0 && act != 1) || (grouped && N % 32 != 0)) : (act != 0 && act != 3)) return -1;
     const dim3 grid((unsigned)((N + (gate ? 7 : 15)) / (gate ? 8 : 16))), block(256);
     const size_t lds = (size_t)M * K * 2;                        // (<= 64 KB)
-#define EVO_PN(MM, G) hipLaunchKernelGGL((postnorm_gemv_kernel<MM, G>), grid, block, lds, (hipStream_t)stream, (const uint4*)y, (const uint4*)g, (const float4*)x, \
-                                         (float4*)x_out, (const uint4*)w, (uint16_t*)out, (int)N, (int)(K / 8), eps, off, grouped ? 1 : 0, (int)act)
+#define EVO_PN(MM, G, S) hipLaunchKernelGGL((postnorm_gemv_kernel<MM, G, S>), grid, block, lds, (hipStream_t)stream, (const uint4*)y, (const uint4*)g,    \
+                                            (const float4*)x, (float4*)x_out, (const uint4*)w, (uint16_t*)out, (int)N, (int)(K / 8), alpha, eps, off, \
+                                            grouped ? 1 : 0, (int)act)
+#define EVO_PN1(MM) do { if (gate) { if (sum) EVO_PN(MM, true, true); else EVO_PN(MM, true, false); }                       \
+                         else { if (sum) EVO_PN(MM, false, true); else EVO_PN(MM, false, false); } } while (0)
     switch (M) {
-        case 1: if (gate) EVO_PN(1, true); else EVO_PN(1, false); break;
-        case 2: if (gate) EVO_PN(2, true); else EVO_PN(2, false); break;
-        case 3: if (gate) EVO_PN(3, true); else EVO_PN(3, false); break;
-        default: if (gate) EVO_PN(4, true); else EVO_PN(4, false); break;
+        case 1: EVO_PN1(1); break;
+        case 2: EVO_PN1(2); break;
+        case 3: EVO_PN1(3); break;
+        default: EVO_PN1(4); break;
     }
+#undef EVO_PN1
 #undef EVO_PN
     return evo_launch_status();
 }
 
 extern "C" int evo_postnorm_linear_small_m_bf16(const void* y, const void* g, const float* x, float* x_out, const void* w, void* z, int64_t M, int64_t N,
-                                                int64_t K, float eps, float w_offset, void* stream) {
-    return postnorm_gemv_launch(y, g, x, x_out, w, z, M, N, K, eps, w_offset, false, 0, 0, stream);
+                                                int64_t K, float alpha, int64_t sum, float eps, float w_offset, int64_t act, void* stream) {
+    return postnorm_gemv_launch(y, g, x, x_out, w, z, M, N, K, alpha, sum != 0, eps, w_offset, false, 0, act, stream);
 }
 
 extern "C" int evo_postnorm_mlp_gate_small_m_bf16(const void* y, const void* g, const float* x, float* x_out, const void* w12, void* a, int64_t M,
-                                                  int64_t I, int64_t K, float eps, float w_offset, int64_t grouped, int64_t act, void* stream) {
-    return postnorm_gemv_launch(y, g, x, x_out, w12, a, M, I, K, eps, w_offset, true, grouped, act, stream);
+                                                  int64_t I, int64_t K, float alpha, int64_t sum, float eps, float w_offset, int64_t grouped,
+                                                  int64_t act, void* stream) {
+    return postnorm_gemv_launch(y, g, x, x_out, w12, a, M, I, K, alpha, sum != 0, eps, w_offset, true, grouped, act, stream);
 }
 
 // ---- 5 <= M <= 16: MFMA form.  Workgroup = 8 waves = 16 output rows; wave w streams its eighth of K:

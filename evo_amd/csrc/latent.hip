@@ -1,6 +1,7 @@
 // Latent attention: keys and values of every head are linear maps of one normed latent c per token, plus one rotated key part shared by
 // all heads; sliding window; one sink per head in the softmax denominator.  Entry points: include/evo_mi355x.h.
-//   prompts:  q | down-projection row -> latent_prep (norm, rotation, cache append) -> k, v of every head by one dense layer -> window_attn
+//   prompts:  q | down-projection row -> latent_prep (norm, rotation, cache append) -> k, v of every head by one dense layer -> window
+//             attention (csrc/window_attn.hip)
 //   decode:   the key map is moved to the query side (q_abs = W_uk^T q), scores and the weighted sum run on the cached latents themselves,
 //             the value map is applied to the one combined latent:  latent_absorb -> latent_decode (split over the window) -> latent_up
 #include "mixers_common.h"
@@ -70,327 +71,6 @@ extern "C" int evo_latent_prep(void* q, int64_t ldq, void* c, void* kr, void* ca
     PrepArgs a = {q, ldq, c, kr, cache, w, inv_freq, pos, seq, cu, (int)H, (int)dn, (int)dr, (int)R, (int)n_rot, (int)ring, (int)rs, eps};
     if (f32) hipLaunchKernelGGL((latent_prep_kernel<float>), dim3((unsigned)M), dim3(256), (size_t)n_rot * 4, (hipStream_t)stream, a);
     else hipLaunchKernelGGL((latent_prep_kernel<uint16_t>), dim3((unsigned)M), dim3(256), (size_t)n_rot * 4, (hipStream_t)stream, a);
-    return evo_launch_status();
-}
-
-// ------------------------------------------------------------------------------------------------ windowed attention of prompts
-struct WinArgs {
-    const void* q; const void* kn; const void* v; const void* kr; void* o;
-    const int* cu_q; const int* cu_k; const float* sink;
-    int64_t ldq, ldkv;                                           // q row pitch; pitch of the kn / v rows
-    int H, dn, dr, dv, window, n_qb;                             // kr rows are dr elements, o rows H dv
-    float scale;
-};
-
-// Matrix-core form (bf16).  A workgroup: 64 QC query rows of one (sequence, head); wave w owns 16 QC of them as MFMA COLUMNS: scores come
-// as S^T = K Q^T (a lane holds one query's scores of four keys per 16-key block), so the softmax needs two cross-lane steps, the
-// probabilities are the next product's operand as they stand (split key order), and O^T = V^T P^T is rescaled by one factor per lane.
-// VEC: every row piece of eight elements is 16-byte aligned.
-template <int KS, int DVB, int QC, bool VEC>
-__global__ __launch_bounds__(256, 2) void window_attn_kernel(WinArgs a, int B) {
-    constexpr int DQ = 32 * KS, PR = DQ + 8, PT = 64 + 4, DVP = 16 * DVB, QB = 64 * QC;
-    constexpr int KG = DQ / 64, VG = DVP / 64;                   // groups of 64 key / value dimensions
-    __shared__ __attribute__((aligned(16))) uint16_t k_rows[64 * PR], v_cols[DVP * PT];
-    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-    const int c16 = lane & 15, g = lane >> 4;
-    // the query blocks of a (sequence, head) share most of their keys: consecutive work items stay on one XCD (block b runs on XCD b % 8)
-    const int per_xcd = gridDim.x >> 3;
-    const int item = (blockIdx.x & 7) * per_xcd + (blockIdx.x >> 3);
-    const int qb = item % a.n_qb, h = item / a.n_qb % a.H, b = item / a.n_qb / a.H;
-    if (b >= B) return;                                          // (the grid is rounded up to a multiple of 8)
-    const int q0 = a.cu_q[b], nq = a.cu_q[b + 1] - q0, k0 = a.cu_k[b], nk = a.cu_k[b + 1] - k0;
-    if (qb * QB >= nq) return;
-    const int off = nk - nq;                                     // key index of query 0
-    const int dh = a.dn + a.dr, dn = a.dn, dv = a.dv;
-    const uint16_t* kr = (const uint16_t*)a.kr + (int64_t)k0 * a.dr;
-    const uint16_t* kn = (const uint16_t*)a.kn + (int64_t)k0 * a.ldkv + (int64_t)h * dn;
-    const uint16_t* vg = (const uint16_t*)a.v + (int64_t)k0 * a.ldkv + (int64_t)h * dv;
-    mx_frag qf[QC][KS];
-    int qi[QC];                                                  // this lane's query of each column block, as a key index
-#pragma unroll
-    for (int c = 0; c < QC; ++c) {
-        const int i = qb * QB + (wave * QC + c) * 16 + c16;
-        qi[c] = i + off;
-        const uint16_t* p = (const uint16_t*)a.q + (int64_t)(q0 + (i < nq ? i : nq - 1)) * a.ldq + (int64_t)h * dh;
-#pragma unroll
-        for (int ks = 0; ks < KS; ++ks) {
-            const int d = 32 * ks + 8 * g;
-            uint4 v = make_uint4(0u, 0u, 0u, 0u);
-            if constexpr (VEC) { if (d < dh) v = *(const uint4*)(p + d); }
-            else {
-                uint32_t w[8];
-#pragma unroll
-                for (int e = 0; e < 8; ++e) w[e] = d + e < dh ? p[d + e] : 0u;
-                v = make_uint4(w[0] | w[1] << 16, w[2] | w[3] << 16, w[4] | w[5] << 16, w[6] | w[7] << 16);
-            }
-            qf[c][ks] = __builtin_bit_cast(mx_frag, v);
-        }
-    }
-    const float sc2 = a.scale * LOG2E;
-    f32x4_t o[QC][DVB];
-    float mx[QC], den[QC];                                       // den: this lane's share (its keys); the sink sits in lane group 0's
-#pragma unroll
-    for (int c = 0; c < QC; ++c) {
-        mx[c] = a.sink[h] * LOG2E;
-        den[c] = g == 0 ? 1.0f : 0.0f;
-#pragma unroll
-        for (int db = 0; db < DVB; ++db) o[c][db] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-    }
-
-    // eight threads share a row: thread (row rt, dims 8 (tid % 8) + 64 i) of keys rt and rt + 32, values of keys 2 rt and 2 rt + 1
-    const int rt = tid >> 3, ct = (tid & 7) * 8;
-    mx_u32x4 rk[KG][2], rv[VG][2];
-    auto any8 = [](const uint16_t* x, int nx, const uint16_t* y, int ny, int d) {       // eight dims of [x (nx) | y (ny) | zeros], any alignment
-        uint32_t w[8];
-#pragma unroll
-        for (int e = 0; e < 8; ++e) w[e] = d + e < nx ? x[d + e] : (d + e < nx + ny ? y[d + e - nx] : 0u);
-        return mx_u32x4{w[0] | w[1] << 16, w[2] | w[3] << 16, w[4] | w[5] << 16, w[6] | w[7] << 16};
-    };
-    // (keys past the end and dimensions past the head's repeat valid ones -- their scores are masked, the queries are zero there, their
-    //  outputs are not stored --, so that the aligned form has no branch among its requests)
-    auto load_k = [&](int j0) __attribute__((always_inline)) {
-#pragma unroll
-        for (int u = 0; u < 2; ++u) {
-            const int j = j0 + rt + 32 * u < nk ? j0 + rt + 32 * u : nk - 1;
-            const uint16_t *pn = kn + j * a.ldkv, *pr_ = kr + (int64_t)j * a.dr;
-#pragma unroll
-            for (int i = 0; i < KG; ++i) {
-                const int d = ct + 64 * i;
-                if constexpr (!VEC) rk[i][u] = any8(pn, dn, pr_, a.dr, d);
-                else {
-                    const int dc = d < dh ? d : dh - 8;
-                    rk[i][u] = *(const mx_u32x4*)(dc < dn ? pn + dc : pr_ + (dc - dn));
-                }
-            }
-        }
-    };
-    auto load_v = [&](int j0) __attribute__((always_inline)) {
-#pragma unroll
-        for (int u = 0; u < 2; ++u) {
-            const int j = j0 + 2 * rt + u < nk ? j0 + 2 * rt + u : nk - 1;
-            const uint16_t* pv = vg + j * a.ldkv;
-#pragma unroll
-            for (int i = 0; i < VG; ++i) {
-                const int d = ct + 64 * i;
-                if constexpr (!VEC) rv[i][u] = any8(pv, dv, pv, 0, d);
-                else rv[i][u] = *(const mx_u32x4*)(pv + (d < dv ? d : dv - 8));
-            }
-        }
-    };
-    auto stage = [&]() __attribute__((always_inline)) {
-#pragma unroll
-        for (int i = 0; i < KG; ++i)
-#pragma unroll
-            for (int u = 0; u < 2; ++u) *(mx_u32x4*)(k_rows + (rt + 32 * u) * PR + ct + 64 * i) = rk[i][u];
-#pragma unroll
-        for (int i = 0; i < VG; ++i)
-#pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                const uint32_t x = rv[i][0][e], y = rv[i][1][e];
-                *(uint32_t*)(v_cols + (ct + 64 * i + 2 * e) * PT + 2 * rt) = (x & 0xffffu) | y << 16;
-                *(uint32_t*)(v_cols + (ct + 64 * i + 2 * e + 1) * PT + 2 * rt) = x >> 16 | (y & 0xffff0000u);
-            }
-    };
-
-    const int last_q = (qb + 1) * QB < nq ? (qb + 1) * QB - 1 : nq - 1;
-    int j_lo = qb * QB + off - a.window + 1;
-    j_lo = j_lo < 0 ? 0 : j_lo & ~63;
-    const int j_hi = last_q + off;                               // last key any row of this block sees
-    const int w_first = qb * QB + wave * QC * 16 + off, w_last = w_first + QC * 16 - 1;   // this wave's queries as key indexes
-    load_k(j_lo);
-    load_v(j_lo);
-    for (int j0 = j_lo; j0 <= j_hi; j0 += 64) {
-        stage();
-        __syncthreads();
-        const bool more = j0 + 64 <= j_hi;
-        const bool mine = j0 <= w_last && j0 + 63 > w_first - a.window;   // some query of this wave sees some key of the tile
-        f32x4_t s[QC][4];
-        if (mine) {
-#pragma unroll
-            for (int jb = 0; jb < 4; ++jb) {
-#pragma unroll
-                for (int c = 0; c < QC; ++c) s[c][jb] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-                for (int ks = 0; ks < KS; ++ks) {
-                    const mx_frag kf = __builtin_bit_cast(mx_frag, *(const uint4*)(k_rows + (16 * jb + c16) * PR + 32 * ks + 8 * g));
-#pragma unroll
-                    for (int c = 0; c < QC; ++c) s[c][jb] = mfma16(kf, qf[c][ks], s[c][jb]);
-                }
-                if (jb & 1) __builtin_amdgcn_sched_barrier(0);   // (bounds the fragments read ahead)
-            }
-        }
-        // the next tile's requests go out in two parts, between the phases: with all of them ahead of the scores the register file spills
-        __builtin_amdgcn_sched_barrier(0);
-        if (more) load_k(j0 + 64);
-        __builtin_amdgcn_sched_barrier(0);
-        mx_frag pf[QC][2];
-        if (mine) {
-            if (j0 + 63 > w_first || j0 <= w_last - a.window) {          // the tile holds an edge of some query's window
-#pragma unroll
-                for (int c = 0; c < QC; ++c)
-#pragma unroll
-                    for (int jb = 0; jb < 4; ++jb)
-#pragma unroll
-                        for (int r = 0; r < 4; ++r) {
-                            const int age = qi[c] - (j0 + 16 * jb + 4 * g + r);
-                            s[c][jb][r] = age >= 0 && age < a.window ? s[c][jb][r] * sc2 : -INFINITY;
-                        }
-            } else {
-#pragma unroll
-                for (int c = 0; c < QC; ++c)
-#pragma unroll
-                    for (int jb = 0; jb < 4; ++jb)
-#pragma unroll
-                        for (int r = 0; r < 4; ++r) s[c][jb][r] *= sc2;
-            }
-#pragma unroll
-            for (int c = 0; c < QC; ++c) {
-                float top = mx[c];
-#pragma unroll
-                for (int jb = 0; jb < 4; ++jb) top = fmaxf(top, fmaxf(fmaxf(s[c][jb][0], s[c][jb][1]), fmaxf(s[c][jb][2], s[c][jb][3])));
-                top = fmaxf(top, __shfl_xor(top, 16, 64));
-                top = fmaxf(top, __shfl_xor(top, 32, 64));
-                if (__builtin_amdgcn_ballot_w64(top > mx[c])) {          // the running maximum moved in some column: rescale
-                    const float f = __builtin_amdgcn_exp2f(mx[c] - top);
-                    mx[c] = top;
-                    den[c] *= f;
-#pragma unroll
-                    for (int db = 0; db < DVB; ++db)
-#pragma unroll
-                        for (int r = 0; r < 4; ++r) o[c][db][r] *= f;
-                }
-                uint32_t w[8];
-#pragma unroll
-                for (int jb = 0; jb < 4; ++jb) {
-                    float e[4];
-#pragma unroll
-                    for (int r = 0; r < 4; ++r) {
-                        e[r] = __builtin_amdgcn_exp2f(s[c][jb][r] - mx[c]);
-                        den[c] += e[r];
-                    }
-                    w[2 * jb] = pack_bf2(e[0], e[1]);
-                    w[2 * jb + 1] = pack_bf2(e[2], e[3]);
-                }
-                pf[c][0] = frag_of(w[0], w[1], w[2], w[3]);
-                pf[c][1] = frag_of(w[4], w[5], w[6], w[7]);
-            }
-        }
-        __builtin_amdgcn_sched_barrier(0);
-        if (more) load_v(j0 + 64);
-        __builtin_amdgcn_sched_barrier(0);
-        if (mine) {
-#pragma unroll
-            for (int jj = 0; jj < 2; ++jj)
-#pragma unroll
-                for (int db = 0; db < DVB; ++db) {
-                    const mx_frag vf = frag_split(v_cols + (16 * db + c16) * PT + 32 * jj + 4 * g);
-#pragma unroll
-                    for (int c = 0; c < QC; ++c) o[c][db] = mfma16(vf, pf[c][jj], o[c][db]);
-                    if ((db & 3) == 3) __builtin_amdgcn_sched_barrier(0);
-                }
-        }
-        __syncthreads();
-    }
-#pragma unroll
-    for (int c = 0; c < QC; ++c) {
-        float l = den[c];
-        l += __shfl_xor(l, 16, 64);
-        l += __shfl_xor(l, 32, 64);
-        const float inv = 1.0f / l;
-        const int i = qi[c] - off;
-        if (i < nq) {
-            uint16_t* op = (uint16_t*)a.o + (int64_t)(q0 + i) * a.H * dv + (int64_t)h * dv;
-#pragma unroll
-            for (int db = 0; db < DVB; ++db) {
-                const int d = 16 * db + 4 * g;
-                if (d + 3 < dv && (dv & 3) == 0)
-                    *(uint2*)(op + d) = make_uint2(pack_bf2(o[c][db][0] * inv, o[c][db][1] * inv), pack_bf2(o[c][db][2] * inv, o[c][db][3] * inv));
-                else {
-#pragma unroll
-                    for (int r = 0; r < 4; ++r)
-                        if (d + r < dv) op[d + r] = f_to_bf(o[c][db][r] * inv);
-                }
-            }
-        }
-    }
-}
-
-// Any sizes, both storage types: one wave per (query, head); lanes are keys for the scores, value columns for the sum
-template <typename T>
-__global__ __launch_bounds__(64) void window_attn_any_kernel(WinArgs a) {
-    extern __shared__ float qs[];                                // dn + dr floats
-    const int qr = blockIdx.x, h = blockIdx.y, b = blockIdx.z, lane = threadIdx.x;
-    const int q0 = a.cu_q[b], nq = a.cu_q[b + 1] - q0, k0 = a.cu_k[b], nk = a.cu_k[b + 1] - k0;
-    if (qr >= nq) return;
-    const int dh = a.dn + a.dr, ki = qr + nk - nq;
-    const T* q = (const T*)a.q + (int64_t)(q0 + qr) * a.ldq + (int64_t)h * dh;
-    for (int d = lane; d < dh; d += 64) qs[d] = ld1(q + d);
-    __syncthreads();
-    const T* kn = (const T*)a.kn + (int64_t)k0 * a.ldkv + (int64_t)h * a.dn;
-    const T* vg = (const T*)a.v + (int64_t)k0 * a.ldkv + (int64_t)h * a.dv;
-    const T* kr = (const T*)a.kr + (int64_t)k0 * a.dr;
-    float m = a.sink[h], l = 1.0f, o[8];
-#pragma unroll
-    for (int e = 0; e < 8; ++e) o[e] = 0.f;
-    for (int j0 = ki - a.window + 1 < 0 ? 0 : ki - a.window + 1; j0 <= ki; j0 += 64) {
-        const int j = j0 + lane;
-        float s = -INFINITY;
-        if (j <= ki) {
-            s = 0.f;
-            for (int d = 0; d < a.dn; ++d) s = fmaf(qs[d], ld1(kn + j * a.ldkv + d), s);
-            for (int d = 0; d < a.dr; ++d) s = fmaf(qs[a.dn + d], ld1(kr + (int64_t)j * a.dr + d), s);
-            s *= a.scale;
-        }
-        const float top = fmaxf(m, wave_max(s)), f = expf(m - top), p = expf(s - top);
-        m = top;
-        l = l * f + wave_sum(p);
-#pragma unroll
-        for (int e = 0; e < 8; ++e) o[e] *= f;
-        const int n = ki - j0 + 1 < 64 ? ki - j0 + 1 : 64;
-        for (int u = 0; u < n; ++u) {
-            const float pu = __shfl(p, u, 64);
-            const T* vr = vg + (j0 + u) * a.ldkv;
-#pragma unroll
-            for (int e = 0; e < 8; ++e)
-                if (lane + 64 * e < a.dv) o[e] = fmaf(pu, ld1(vr + lane + 64 * e), o[e]);
-        }
-    }
-    T* op = (T*)a.o + (int64_t)(q0 + qr) * a.H * a.dv + (int64_t)h * a.dv;
-#pragma unroll
-    for (int e = 0; e < 8; ++e)
-        if (lane + 64 * e < a.dv) st1(op + lane + 64 * e, o[e] / l);
-}
-
-extern "C" int evo_window_attn(const void* q, int64_t ldq, const void* kn, const void* v, int64_t ldkv, const void* kr, void* o, const int* cu_q,
-                               const int* cu_k, const float* sink, int64_t B, int64_t H, int64_t dn, int64_t dr, int64_t dv, int64_t window,
-                               int64_t max_q, float scale, int64_t f32, int64_t mfma, void* stream) {
-    if (!q || !kn || !v || !kr || !o || !cu_q || !cu_k || !sink || B <= 0 || B > 65535 || H <= 0 || H > 65535) return -1;
-    if (dn < 0 || dr < 0 || dn + dr <= 0 || dn + dr > 8192 || dv <= 0 || dv > 512 || window <= 0 || max_q <= 0 || max_q > 0x3fffffff) return -1;
-    if (ldq < H * (dn + dr) || ldkv < H * dv) return -1;
-    const int w = window > 0x3fffffff ? 0x3fffffff : (int)window;
-    WinArgs a = {q, kn, v, kr, o, cu_q, cu_k, sink, ldq, ldkv, (int)H, (int)dn, (int)dr, (int)dv, w, 0, scale};
-    hipStream_t s = (hipStream_t)stream;
-    const int64_t dq = dn + dr;
-    if (!f32 && mfma && dq <= 256 && dv <= 256) {
-        const bool vec = dn % 8 == 0 && dr % 8 == 0 && dv % 8 == 0 && ldq % 8 == 0 && ldkv % 8 == 0 &&
-                         (((uintptr_t)q | (uintptr_t)kn | (uintptr_t)v | (uintptr_t)kr) & 15) == 0;
-#define WA(KS, DVB, QC, VEC)                                                                                               \
-    do {                                                                                                                   \
-        a.n_qb = (int)((max_q + 64 * QC - 1) / (64 * QC));                                                                 \
-        const int64_t items = (int64_t)a.n_qb * H * B;                                                                     \
-        if (items > 0x7ffffff0) return -1;                                                                                 \
-        hipLaunchKernelGGL((window_attn_kernel<KS, DVB, QC, VEC>), dim3((unsigned)((items + 7) / 8 * 8)), dim3(256), 0, s, a, (int)B); \
-    } while (0)
-#define WAV(KS, QC) do { if (dv <= 64) WA(KS, 4, QC, true); else if (dv <= 128) WA(KS, 8, QC, true); else WA(KS, 16, 1, true); } while (0)
-        if (!vec) { if (dq <= 64 && dv <= 64) WA(2, 4, 2, false); else WA(8, 16, 1, false); }
-        else if (dq <= 64) WAV(2, 2); else if (dq <= 128) WAV(4, 2); else if (dq <= 192) WAV(6, 2); else WAV(8, 1);
-#undef WAV
-#undef WA
-        return evo_launch_status();
-    }
-    const dim3 grid((unsigned)max_q, (unsigned)H, (unsigned)B);
-    if (f32) hipLaunchKernelGGL((window_attn_any_kernel<float>), grid, dim3(64), (size_t)dq * 4, s, a);
-    else hipLaunchKernelGGL((window_attn_any_kernel<uint16_t>), grid, dim3(64), (size_t)dq * 4, s, a);
     return evo_launch_status();
 }
 

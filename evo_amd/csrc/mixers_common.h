@@ -1,4 +1,4 @@
-// Shared helpers of the mixer kernels (csrc/stream.hip, csrc/lightning.hip, csrc/latent.hip): element access for the two storage types
+// Shared helpers of the mixer kernels (csrc/{stream,window_attn,lightning,latent,heads,rglru}.hip): element access for the two storage types
 // (bf16 words, fp32), block reductions, and the hi / lo split of an fp32 operand for the matrix cores.
 #pragma once
 #include "common.h"
@@ -47,6 +47,17 @@ template <> __device__ __forceinline__ float sigmoid_t<uint16_t>(float z) {
     return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(z * -1.4426950408889634f));
 }
 template <typename T> __device__ __forceinline__ float silu_t(float z) { return z * sigmoid_t<T>(z); }
+
+// tanh-form GELU: z times the logistic of 2 sqrt(2 / pi) (z + 0.044715 z^3)
+template <typename T> __device__ __forceinline__ float gelu_tanh_t(float z) { return z * sigmoid_t<T>(1.5957691216057308f * fmaf(0.044715f * z * z, z, z)); }
+
+// activations by code: 1 SiLU, 2 tanh-form GELU, 3 square of relu
+template <typename T> __device__ __forceinline__ float act_t(float z, int act) {
+    if (act == 1) return silu_t<T>(z);
+    if (act == 2) return gelu_tanh_t<T>(z);
+    z = fmaxf(z, 0.f);
+    return z * z;
+}
 
 // base^m for m >= 0 from log2(base) (-inf for base 0)
 __device__ __forceinline__ float pow_log2(float l2, int m) { return m == 0 ? 1.0f : exp2f(l2 * (float)m); }

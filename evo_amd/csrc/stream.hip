@@ -1,5 +1,5 @@
 // Token-local kernels of models whose residual stream is kept in fp32: scaled embedding, the norm of a sublayer's output added to the
-// stream, the final norm, the gated norm behind a linear-attention mixer, the gate of a gated MLP.  One workgroup per row, fp32 math,
+// stream, the norm of their sum, the final norm, the gated norm behind a linear-attention mixer, the gate of a gated MLP.  One workgroup per row, fp32 math,
 // one rounding on the way out; storage type T is bf16 or fp32.  Entry points: include/evo_mi355x.h.
 #include "mixers_common.h"
 #include "../../include/evo_mi355x.h"
@@ -46,11 +46,12 @@ extern "C" int evo_embed_stream(const int64_t* ids, const void* w, float* x, voi
 }
 
 // ---------------------------------------------------------------------------------------------- x += norm(y) * (off + w)
+// SUM: x = norm(alpha x + y) * (off + w); `y` below is then the sum.
 // y stays in registers between the two passes (rows up to 4,096 elements); x is written in fp32 and, for the next sublayer's matrix
 // product, once more in bf16.
-template <typename T, int V>
-__global__ __launch_bounds__(256) void postnorm_residual_kernel(const void* __restrict__ y_, const void* __restrict__ w_, float* __restrict__ x,
-                                                                uint16_t* __restrict__ xb, int D, float eps, float off) {
+template <typename T, int V, bool SUM>
+__device__ __forceinline__ void closing_norm(const void* __restrict__ y_, const void* __restrict__ w_, float* __restrict__ x,
+                                             uint16_t* __restrict__ xb, int D, float alpha, float eps, float off) {
     constexpr int KEEP = V == 8 ? 2 : 4;                         // runs of V elements a thread keeps in registers (D <= 256 V KEEP)
     __shared__ float red[4];
     const T* w = (const T*)w_;
@@ -58,18 +59,27 @@ __global__ __launch_bounds__(256) void postnorm_residual_kernel(const void* __re
     const T* y = (const T*)y_ + row * D;
     float keep[KEEP][V];
     float ss = 0.f;
+    auto load = [&](int c, float* f) {
+        vec_io<T, V>::load(y + c, f);
+        if constexpr (SUM) {
+            float r[V];
+            vec_io<float, V>::load(x + row * D + c, r);
+#pragma unroll
+            for (int e = 0; e < V; ++e) f[e] = fmaf(alpha, r[e], f[e]);
+        }
+    };
 #pragma unroll
     for (int i = 0; i < KEEP; ++i) {
         const int c = (threadIdx.x + 256 * i) * V;
         if (c < D) {
-            vec_io<T, V>::load(y + c, keep[i]);
+            load(c, keep[i]);
 #pragma unroll
             for (int e = 0; e < V; ++e) ss = fmaf(keep[i][e], keep[i][e], ss);
         }
     }
     for (int c = (threadIdx.x + 256 * KEEP) * V; c < D; c += 256 * V) {
         float f[V];
-        vec_io<T, V>::load(y + c, f);
+        load(c, f);
 #pragma unroll
         for (int e = 0; e < V; ++e) ss = fmaf(f[e], f[e], ss);
     }
@@ -77,9 +87,9 @@ __global__ __launch_bounds__(256) void postnorm_residual_kernel(const void* __re
     auto finish = [&](int c, const float* f) {
         float g[V], r[V];
         vec_io<T, V>::load(w + c, g);
-        vec_io<float, V>::load(x + row * D + c, r);
+        if constexpr (!SUM) vec_io<float, V>::load(x + row * D + c, r);
 #pragma unroll
-        for (int e = 0; e < V; ++e) r[e] += f[e] * inv * (off + g[e]);
+        for (int e = 0; e < V; ++e) r[e] = SUM ? f[e] * inv * (off + g[e]) : fmaf(f[e] * inv, off + g[e], r[e]);
         vec_io<float, V>::store(x + row * D + c, r);
         if (xb) vec_io<uint16_t, V>::store(xb + row * D + c, r);
     };
@@ -90,9 +100,20 @@ __global__ __launch_bounds__(256) void postnorm_residual_kernel(const void* __re
     }
     for (int c = (threadIdx.x + 256 * KEEP) * V; c < D; c += 256 * V) {
         float f[V];
-        vec_io<T, V>::load(y + c, f);
+        load(c, f);
         finish(c, f);
     }
+}
+
+template <typename T, int V>
+__global__ __launch_bounds__(256) void postnorm_residual_kernel(const void* __restrict__ y, const void* __restrict__ w, float* __restrict__ x,
+                                                                uint16_t* __restrict__ xb, int D, float eps, float off) {
+    closing_norm<T, V, false>(y, w, x, xb, D, 1.f, eps, off);
+}
+template <typename T, int V>
+__global__ __launch_bounds__(256) void sum_norm_kernel(const void* __restrict__ y, const void* __restrict__ w, float* __restrict__ x,
+                                                       uint16_t* __restrict__ xb, int D, float alpha, float eps, float off) {
+    closing_norm<T, V, true>(y, w, x, xb, D, alpha, eps, off);
 }
 
 extern "C" int evo_postnorm_residual(const void* y, const void* w, float* x, void* xb, int64_t M, int64_t D, float eps, float w_offset,
@@ -100,6 +121,13 @@ extern "C" int evo_postnorm_residual(const void* y, const void* w, float* x, voi
     if (M < 0 || M > 0x7fffffff || D <= 0 || D > 0x3fffffff) return -1;
     if (M == 0) return 0;
     STREAM_DISPATCH(postnorm_residual_kernel, D % 8 == 0, (unsigned)M, y, w, x, (uint16_t*)xb, (int)D, eps, w_offset);
+}
+
+extern "C" int evo_sum_norm(const void* y, const void* w, float* x, void* xb, int64_t M, int64_t D, float alpha, float eps, float w_offset,
+                            int64_t f32, void* stream) {
+    if (!y || !w || !x || M < 0 || M > 0x7fffffff || D <= 0 || D > 0x3fffffff) return -1;
+    if (M == 0) return 0;
+    STREAM_DISPATCH(sum_norm_kernel, D % 8 == 0, (unsigned)M, y, w, x, (uint16_t*)xb, (int)D, alpha, eps, w_offset);
 }
 
 // ---------------------------------------------------------------------------------------------- out = norm(x) * (off + w), x the stream
@@ -218,9 +246,9 @@ extern "C" int evo_silu_gate(const void* z, void* a, int64_t M, int64_t I, int64
     STREAM_DISPATCH(silu_gate_kernel, I % 8 == 0, grid, z, a, M, I);
 }
 
-// ---------------------------------------------------------------------------------------------- z[:, :n] = silu(z[:, :n]) in place
+// ---------------------------------------------------------------------------------------------- z[:, :n] = act(z[:, :n]) in place
 template <typename T, int V>
-__global__ __launch_bounds__(256) void silu_cols_kernel(void* __restrict__ z_, int64_t ld, int64_t M, int64_t n) {
+__global__ __launch_bounds__(256) void act_cols_kernel(void* __restrict__ z_, int64_t ld, int64_t M, int64_t n, int act) {
     T* z = (T*)z_;
     const int64_t per = n / V, total = M * per;
     for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < total; i += (int64_t)gridDim.x * 256) {
@@ -229,16 +257,16 @@ __global__ __launch_bounds__(256) void silu_cols_kernel(void* __restrict__ z_, i
         float f[V];
         vec_io<T, V>::load(p, f);
 #pragma unroll
-        for (int e = 0; e < V; ++e) f[e] = silu_t<T>(f[e]);
+        for (int e = 0; e < V; ++e) f[e] = act_t<T>(f[e], act);
         vec_io<T, V>::store(p, f);
     }
 }
 
-extern "C" int evo_silu_cols(void* z, int64_t ld, int64_t M, int64_t n, int64_t f32, void* stream) {
-    if (M < 0 || n <= 0 || ld < n) return -1;
+extern "C" int evo_act_cols(void* z, int64_t ld, int64_t M, int64_t n, int64_t act, int64_t f32, void* stream) {
+    if (M < 0 || n <= 0 || ld < n || act < 1 || act > 3) return -1;
     if (M == 0) return 0;
     const bool vec = n % 8 == 0 && ld % 8 == 0 && ((uintptr_t)z & 15) == 0;
     const int64_t total = M * (vec ? n / 8 : n);
     const unsigned grid = (unsigned)((total + 255) / 256 < 16384 ? (total + 255) / 256 : 16384);
-    STREAM_DISPATCH(silu_cols_kernel, vec, grid, z, ld, M, n);
+    STREAM_DISPATCH(act_cols_kernel, vec, grid, z, ld, M, n, (int)act);
 }

@@ -15,13 +15,14 @@ import re
 import torch
 import yaml
 
+from .batodra import Batodra
 from .sh.model import StripedHyena
 from .sh.utils import dotdict
 from .tokenizer import CharLevelTokenizer
 from .vozalorn import Vozalorn
 
 # model classes by the `architecture` a config names (none: StripedHyena)
-ARCHITECTURES = {"StripedHyena": StripedHyena, "Vozalorn": Vozalorn}
+ARCHITECTURES = {"StripedHyena": StripedHyena, "Vozalorn": Vozalorn, "Batodra": Batodra}
 
 MODEL_NAMES = [
     "evo-1.5-8k-base",

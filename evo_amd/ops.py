@@ -64,20 +64,27 @@ _SIGNATURES = {
     "evo_gated_norm": ([_PTR] * 2 + [_I64] + [_PTR] * 2 + [_I64] * 2 + [_F32, _I64, _PTR], _c.c_int),
     "evo_silu_gate": ([_PTR] * 2 + [_I64] * 3 + [_PTR], _c.c_int),
     "evo_lightning_chunk_bf16": ([_PTR, _I64] + [_PTR] * 6 + [_I64] * 6 + [_PTR], _c.c_int),
-    "evo_postnorm_linear_small_m_bf16": ([_PTR] * 6 + [_I64] * 3 + [_F32] * 2 + [_PTR], _c.c_int),
-    "evo_postnorm_mlp_gate_small_m_bf16": ([_PTR] * 6 + [_I64] * 3 + [_F32] * 2 + [_I64] * 2 + [_PTR], _c.c_int),
-    "evo_silu_cols": ([_PTR] + [_I64] * 4 + [_PTR], _c.c_int),
-    "evo_linear_silu_mfma_bf16": ([_PTR] * 3 + [_I64] * 4 + [_PTR], _c.c_int),
+    "evo_postnorm_linear_small_m_bf16": ([_PTR] * 6 + [_I64] * 3 + [_F32, _I64] + [_F32] * 2 + [_I64, _PTR], _c.c_int),
+    "evo_postnorm_mlp_gate_small_m_bf16": ([_PTR] * 6 + [_I64] * 3 + [_F32, _I64] + [_F32] * 2 + [_I64] * 2 + [_PTR], _c.c_int),
+    "evo_sum_norm": ([_PTR] * 4 + [_I64] * 2 + [_F32] * 3 + [_I64, _PTR], _c.c_int),
+    "evo_act_cols": ([_PTR] + [_I64] * 5 + [_PTR], _c.c_int),
+    "evo_linear_act_mfma_bf16": ([_PTR] * 4 + [_I64] * 5 + [_PTR], _c.c_int),
     "evo_lightning_recurrent": ([_PTR, _I64] + [_PTR] * 5 + [_I64] * 6 + [_PTR], _c.c_int),
     "evo_latent_prep": ([_PTR, _I64] + [_PTR] * 8 + [_I64] * 8 + [_F32, _I64, _PTR], _c.c_int),
-    "evo_window_attn": ([_PTR, _I64, _PTR, _PTR, _I64] + [_PTR] * 5 + [_I64] * 7 + [_F32] + [_I64] * 2 + [_PTR], _c.c_int),
+    "evo_window_attn": ([_PTR, _I64, _PTR, _PTR, _I64] + [_PTR] * 5 + [_I64] * 10 + [_F32] * 4 + [_I64] * 2 + [_PTR], _c.c_int),
+    "evo_heads_prep": ([_PTR, _I64] + [_PTR] * 7 + [_I64] * 9 + [_F32] * 2 + [_I64] * 2 + [_PTR], _c.c_int),
+    "evo_heads_decode": ([_PTR, _I64] + [_PTR] * 4 + [_I64] * 9 + [_F32] + [_I64] * 2 + [_PTR], _c.c_int),
+    "evo_heads_merge": ([_PTR] * 3 + [_I64] * 5 + [_F32] * 3 + [_I64, _PTR], _c.c_int),
+    "evo_rglru_chunk_bf16": ([_PTR, _I64] + [_PTR] * 13 + [_I64] * 6 + [_PTR], _c.c_int),
+    "evo_rglru_step_bf16": ([_PTR, _I64] + [_PTR] * 11 + [_I64] * 5 + [_PTR], _c.c_int),
+    "evo_rglru_any": ([_PTR, _I64] + [_PTR] * 15 + [_I64] * 7 + [_PTR], _c.c_int),
     "evo_latent_absorb": ([_PTR, _I64] + [_PTR] * 2 + [_I64] * 7 + [_PTR], _c.c_int),
     "evo_latent_decode": ([_PTR] * 5 + [_I64] * 8 + [_F32] + [_I64] * 2 + [_PTR], _c.c_int),
     "evo_latent_up": ([_PTR] * 5 + [_I64] * 7 + [_PTR], _c.c_int),
 }
 
 _LIB = None
-ABI_VERSION = 11         # must equal EVO_ABI_VERSION in include/evo_mi355x.h (bumped on every signature change)
+ABI_VERSION = 12         # must equal EVO_ABI_VERSION in include/evo_mi355x.h (bumped on every signature change)
 
 
 class EvoLibraryError(RuntimeError):

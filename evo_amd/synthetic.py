@@ -13,7 +13,7 @@ def synthetic_state_dict(model, seed: int = 0, device=None, profile: str = "defa
     `profile="contractive"`: the same draw, then the output projections of blocks 1.. rescaled so that a block's update of the
     residual stream is ~7 % of the stream's norm (calibrate_contractive below) -- what trained residual stacks look like."""
     if hasattr(model, "tensor_shapes"):
-        return shaped_state_dict(model.tensor_shapes(), seed, device)
+        return shaped_state_dict(model.tensor_shapes(), seed, device, 1.0 - model.NORM_OFFSET)
     if profile not in ("default", "contractive"):
         raise ValueError(f"unknown synthetic weight profile {profile!r}")
     if profile == "contractive":
@@ -70,16 +70,16 @@ def synthetic_state_dict(model, seed: int = 0, device=None, profile: str = "defa
     return sd
 
 
-def shaped_state_dict(shapes: Dict[str, tuple], seed: int = 0, device=None) -> Dict[str, torch.Tensor]:
+def shaped_state_dict(shapes: Dict[str, tuple], seed: int = 0, device=None, norm_one: float = 0.0) -> Dict[str, torch.Tensor]:
     """Random bf16 weights for a model that lists its tensors: matrices N(0, 1 / fan-in), vectors N(0, 0.3) (around one for the plain norms
-    inside a mixer)."""
+    inside a mixer, around `norm_one` for the norms outside)."""
     device = torch.device(device) if device is not None else torch.device("cpu")
     g = torch.Generator(device=device).manual_seed(seed)
     out = {}
     for name, shape in shapes.items():
         t = torch.randn(*shape, generator=g, device=device, dtype=torch.float32)
         if len(shape) == 1:
-            t = t * 0.3 + (1.0 if ".mix." in name and name.endswith("norm") else 0.0)
+            t = t * 0.3 + ((1.0 if ".mix." in name else norm_one) if "norm" in name else 0.0)
         elif name != "embed":
             t = t / math.sqrt(shape[1])
         out[name] = t.to(torch.bfloat16)

@@ -50,8 +50,11 @@ extern "C" {
  *      takes up to 64 rows and an optional workspace (`ws`, `ws_bytes`: split over K across workgroups for the narrow layers); evo_hyena_ct gained `y_row_pitch` (rows of y between two batch rows: the scoring path runs the 512 k main tokens
  *      of every row through the operator and the one token behind them through the single-token launch, see below).
  *  11: evo_mlp_gate_mfma_bf16 and evo_mlp_gate_small_m_bf16 gained `act` (gate function: 0 exact-erf GELU, 1 SiLU); evo_linear_silu_mfma_bf16, the evo_postnorm_* launches and the mixers library added:
- *      fp32-residual-stream kernels, decayed linear attention, latent attention (the last section of this file). */
-#define EVO_ABI_VERSION 11
+ *      fp32-residual-stream kernels, decayed linear attention, latent attention (the last section of this file).
+ *  12: evo_linear_act_mfma_bf16 (bias, three activations) and evo_act_cols take the places of evo_linear_silu_mfma_bf16 and evo_silu_cols; the
+ *      evo_postnorm_* launches gained the norm of the sum (`alpha`, `sum`) and the plain one an activation; evo_window_attn gained grouped key heads,
+ *      kept first tokens and two maps; evo_sum_norm, evo_heads_* and evo_rglru_* added. */
+#define EVO_ABI_VERSION 12
 int evo_abi_version(void);
 
 /* ---- embedding gather ------------------------------------------------------------------------
@@ -257,9 +260,10 @@ int evo_linear_small_m_bf16(const void* x, const void* w, const void* bias, cons
 int evo_linear_mfma_bf16(const void* x, const void* w, const void* bias, const void* residual, void* y,
                          int64_t M, int64_t N, int64_t K, void* stream);
 
-/* ... with SiLU on columns [0, act_cols) of the result (before its one rounding) and none behind them: the input projection of a
- * linear-attention mixer.  act_cols % 256 == 0, K >= 128, otherwise the contract of evo_linear_mfma_bf16. */
-int evo_linear_silu_mfma_bf16(const void* x, const void* w, void* y, int64_t M, int64_t N, int64_t K, int64_t act_cols, void* stream);
+/* ... with an activation on columns [0, act_cols) of the result (before its one rounding) and none behind them; act 1: SiLU, 2: GELU (tanh
+ * form), 3: square of relu; bias [N] or NULL.  act_cols % 256 == 0, K >= 128, otherwise the contract of evo_linear_mfma_bf16. */
+int evo_linear_act_mfma_bf16(const void* x, const void* w, const void* bias, void* y, int64_t M, int64_t N, int64_t K, int64_t act_cols,
+                             int64_t act, void* stream);
 
 /* ---- gated MLP, first half, on the MFMA pipe (prefill) ----------------------------------------------------------
  * replaces l1 / l2 (two nn.Linear GEMMs) + F.gelu + the elementwise product of ParallelGatedMLP.forward
@@ -336,13 +340,15 @@ int evo_norm_mlp_gate_small_m_bf16(const void* x, const void* scale, const void*
                                    int64_t K, float eps, int64_t grouped, void* stream);
 
 /* ---- a sublayer's closing norm folded into the next layer (decode form of models with an fp32 residual stream) ----------------
- * x_out = x + y / sqrt(mean(y^2) + eps) * (w_offset + g), fp32 [M, K] (x_out is another buffer than x), and on its bf16 rounding
- *   z [M, N] = x_out . w^T        or        a [M, I] = act(x_out . W1^T) * (x_out . W2^T)   (w12, grouped, act as in evo_mlp_gate_small_m_bf16)
+ * x_out = x + y / sqrt(mean(y^2) + eps) * (w_offset + g)                                         (sum 0), or
+ * x_out = t / sqrt(mean(t^2) + eps) * (w_offset + g), t = alpha x + y                              (sum 1),
+ * fp32 [M, K] (x_out is another buffer than x), and on its bf16 rounding
+ *   z [M, N] = x_out . w^T, through the square of relu with act 3 (0: none), or        a [M, I] = act(x_out . W1^T) * (x_out . W2^T)   (w12, grouped, act as in evo_mlp_gate_small_m_bf16)
  * y [M, K], g [K] bf16; 1 <= M <= 4, K % 8 == 0, K <= 8192. */
 int evo_postnorm_linear_small_m_bf16(const void* y, const void* g, const float* x, float* x_out, const void* w, void* z, int64_t M, int64_t N,
-                                     int64_t K, float eps, float w_offset, void* stream);
+                                     int64_t K, float alpha, int64_t sum, float eps, float w_offset, int64_t act, void* stream);
 int evo_postnorm_mlp_gate_small_m_bf16(const void* y, const void* g, const float* x, float* x_out, const void* w12, void* a, int64_t M, int64_t I,
-                                       int64_t K, float eps, float w_offset, int64_t grouped, int64_t act, void* stream);
+                                       int64_t K, float alpha, int64_t sum, float eps, float w_offset, int64_t grouped, int64_t act, void* stream);
 
 /* ---- gated MLP activation ---------------------------------------------------------------------------
  * replaces ATen gelu + mul                                  [REF evo/configs/evo-1-8k-base_inference.yml:38]
@@ -378,8 +384,8 @@ int evo_unembed_logprob_bf16(const void* hidden, const void* emb, const int64_t*
 int evo_probe_copy_f4(const void* src, void* dst, int64_t nbytes, void* stream);
 int evo_probe_mfma_bf16(float* out, int64_t n_blocks, int64_t iters, void* stream);
 
-/* ==== mixers library (libevo_mi355x_mixers.so) =========================================================================
- * Kernels of the models that a config.json describes layer by layer (evo_amd/vozalorn.py).  The residual stream x [M, D] is fp32; `f32`
+/* ==== mixers (libevo_mi355x_mixers.so, _latent, _lightning, _heads, _rglru) =========================================================================
+ * Kernels of the models that a config.json describes layer by layer (evo_amd/decoder.py).  The residual stream x [M, D] is fp32; `f32`
  * selects the storage type of everything passed as void* (0: bf16, 1: fp32), math is fp32.  Tokens of a batch are packed: sequence b owns
  * rows cu[b] .. cu[b + 1] - 1 (int32, B + 1 entries).  Any sizes unless stated. */
 
@@ -389,6 +395,9 @@ int evo_embed_stream(const int64_t* ids, const void* w, float* x, void* xb, int6
 /* x += y / sqrt(mean(y^2) + eps) * (w_offset + w), in place, and the bf16 copy xb of the new x (NULL: not wanted). */
 int evo_postnorm_residual(const void* y, const void* w, float* x, void* xb, int64_t M, int64_t D, float eps, float w_offset, int64_t f32,
                           void* stream);
+/* x <- t / sqrt(mean(t^2) + eps) * (w_offset + w) with t = alpha * x + y, in place, and the bf16 copy xb of the new x (NULL: not wanted). */
+int evo_sum_norm(const void* y, const void* w, float* x, void* xb, int64_t M, int64_t D, float alpha, float eps, float w_offset, int64_t f32,
+                 void* stream);
 /* out = x / sqrt(mean(x^2) + eps) * (w_offset + w) */
 int evo_rmsnorm_stream(const float* x, const void* w, void* out, int64_t M, int64_t D, float eps, float w_offset, int64_t f32, void* stream);
 /* out = o / sqrt(mean(o^2) + eps) * w * sigmoid(g); g rows have pitch ldg. */
@@ -396,8 +405,8 @@ int evo_gated_norm(const void* o, const void* g, int64_t ldg, const void* w, voi
                    void* stream);
 /* a [M, I] = silu(z[:, :I]) * z[:, I:] */
 int evo_silu_gate(const void* z, void* a, int64_t M, int64_t I, int64_t f32, void* stream);
-/* z[:, :n] = silu(z[:, :n]) in place, rows of pitch ld */
-int evo_silu_cols(void* z, int64_t ld, int64_t M, int64_t n, int64_t f32, void* stream);
+/* z[:, :n] = act(z[:, :n]) in place, rows of pitch ld; act 1: SiLU, 2: GELU (tanh form), 3: square of relu */
+int evo_act_cols(void* z, int64_t ld, int64_t M, int64_t n, int64_t act, int64_t f32, void* stream);
 
 /* ---- linear attention with a constant decay per head: S_t = a_h S_{t-1} + k_t v_t^T, o_t = S_t^T q_t ------------------------------
  * z rows (pitch ld) start with [q (H dk) | k (H dk) | v (H dv)] after their SiLU; o [M, H dv]; state [B, H, dk, dv] fp32 (may be NULL:
@@ -411,6 +420,58 @@ int evo_lightning_chunk_bf16(const void* z, int64_t ld, void* o, float* state, f
 int evo_lightning_recurrent(const void* z, int64_t ld, void* o, float* state, const float* decay, const int* cu, const int* resume, int64_t B,
                             int64_t H, int64_t dk, int64_t dv, int64_t act, int64_t f32, void* stream);
 
+/* ---- softmax attention of packed prompts --------------------------------------------------------------------------------
+ * o_i = sum_j p_ij v_j over the visible keys, p = exp(scale q.k) / (sum exp(scale q.k) [+ exp(sink)]).  A sequence's queries are the LAST
+ * cu_q lengths of its cu_k keys; key j is visible to query i (indexes among the keys) when j <= i and (i - j < window or j < keep): a sliding
+ * window whose first `keep` tokens stay visible.  H query heads share kv_heads key / value heads.  Per head q = [dn | dr] (pitch ldq), k =
+ * [kn (dn) | kr (dr, one for all heads; NULL with dr = 0)], v (dv); kn and v rows have pitch ldkv, o is [Mq, H dv].  sink [H] or NULL.
+ * maps 2 (differential attention; dr = 0, no sink): rows of q and kn hold [map 1 | map 2] per head, v is shared, and
+ *   o = gain * d / sqrt(mean(d^2) + eps),  d = o_map1 - lam * o_map2     (the mean runs over the head's dv values)
+ * dv <= 512.  mfma 0: the any-size kernel (also taken for fp32 and beyond 256 -- two maps: 128 -- key or 256 value dimensions). */
+int evo_window_attn(const void* q, int64_t ldq, const void* kn, const void* v, int64_t ldkv, const void* kr, void* o, const int* cu_q,
+                    const int* cu_k, const float* sink, int64_t B, int64_t H, int64_t kv_heads, int64_t maps, int64_t dn, int64_t dr, int64_t dv,
+                    int64_t window, int64_t keep, int64_t max_q, float scale, float lam, float gain, float eps, int64_t f32, int64_t mfma, void* stream);
+
+/* ---- attention with cached keys and values (csrc/heads.hip) ---------------------------------------------------------------
+ * evo_heads_prep: row m of z (pitch ld) = [nq query vectors | nk key vectors (dim each) | nv values].  In place, per query and key vector:
+ * RMS norm with weight qw / kw (NULL: none), rotation of the pairs (i, i + n_rot / 2) by pos[m] * inv_freq[i] with cosine and sine times amp,
+ * division by the root mean square (unit != 0).  Keys and values also go to the sequence's cache [rows, ring, rs] (NULL: none) as [keys |
+ * values]: token p sits at slot p for p < keep, else at keep + (p - keep) % (ring - keep).  seq [M]: sequence of a row (NULL: row m); cu:
+ * of a sequence's tokens only the first `keep` positions and the last ring - keep tokens are cached (NULL: all are). */
+int evo_heads_prep(void* z, int64_t ld, void* cache, const void* qw, const void* kw, const float* inv_freq, const int64_t* pos, const int* seq,
+                   const int* cu, int64_t M, int64_t nq, int64_t nk, int64_t dim, int64_t nv, int64_t n_rot, int64_t keep, int64_t ring, int64_t rs,
+                   float amp, float eps, int64_t unit, int64_t f32, void* stream);
+/* Decode, one query per sequence (row b of z, position pos[b], its token already in the cache): every slot written so far is visible.
+ * evo_heads_decode: n_split partial softmax sums (part_o [B, H maps, n_split, dv] unnormalised, part_ml [B, H maps, n_split, 2] = running max in
+ * the log2 domain, denominator); mfma 0: the any-size kernel.  evo_heads_merge: o [B, H dv] of the merged parts; maps 2: as in
+ * evo_window_attn.  dv <= 512. */
+int evo_heads_decode(const void* z, int64_t ld, const void* cache, const int64_t* pos, float* part_o, float* part_ml, int64_t B, int64_t H,
+                     int64_t kv_heads, int64_t maps, int64_t dim, int64_t dv, int64_t ring, int64_t rs, int64_t n_split, float scale, int64_t f32,
+                     int64_t mfma, void* stream);
+int evo_heads_merge(const float* part_o, const float* part_ml, void* o, int64_t B, int64_t H, int64_t maps, int64_t dv, int64_t n_split, float lam,
+                    float gain, float eps, int64_t f32, void* stream);
+
+/* ---- gated linear recurrence behind a short convolution (csrc/rglru.hip) ---------------------------------------------------
+ * z rows (pitch ld) start with [y (W) | x (W)]; in_b [2 W] or NULL is added to them first; y still needs its tanh-GELU when act != 0.
+ *   u = conv(x) + conv_b     (conv [W, taps], last column the current token, zeros before a sequence's start)
+ *   r = sigmoid(ra_n u_n + ra_b), i = sigmoid(ri_n u_n + ri_b) in each of nb blocks of bs = W / nb channels (ra, ri [nb, bs, bs])
+ *   a = exp(decay r), S <- a S + sqrt(1 - a^2) i u,  o = S y             (decay [W] fp32: -c softplus(lambda), at most 0)
+ * state [rows, 1 + taps, W] fp32 (may be NULL: nothing is kept): row 0 is S, row 1 + p % taps the x of position p; read where resume[b] != 0
+ * (resume NULL: every sequence starts from zero), left after the last token.  pos [M]: position of every row's token.
+ * evo_rglru_chunk_bf16: prompts on the matrix cores; bs % 8 == 0, bs <= 384, taps <= 4, in_b NULL and y activated by the caller; seg_len % 64 == 0;
+ *   seg [B, ceil(max_len / seg_len), 2, W] fp32 workspace, needed when there is more than one segment.
+ * evo_rglru_step_bf16: one token per sequence (row b), same sizes, updates state[b] in place.
+ * evo_rglru_any: any sizes, both storage types; ab [M, 2, W] fp32 workspace; cu NULL: one token per sequence. */
+int evo_rglru_chunk_bf16(const void* z, int64_t ld, void* o, float* state, float* seg, const void* conv, const void* conv_b, const void* ra,
+                         const void* ra_b, const void* ri, const void* ri_b, const float* decay, const int64_t* pos, const int* cu, const int* resume,
+                         int64_t B, int64_t W, int64_t nb, int64_t taps, int64_t max_len, int64_t seg_len, void* stream);
+int evo_rglru_step_bf16(const void* z, int64_t ld, const void* in_b, void* o, float* state, const void* conv, const void* conv_b, const void* ra,
+                        const void* ra_b, const void* ri, const void* ri_b, const float* decay, const int64_t* pos, int64_t B, int64_t W, int64_t nb,
+                        int64_t taps, int64_t act, void* stream);
+int evo_rglru_any(const void* z, int64_t ld, const void* in_b, void* o, float* state, float* ab, const void* conv, const void* conv_b, const void* ra,
+                  const void* ra_b, const void* ri, const void* ri_b, const float* decay, const int64_t* pos, const int* seq, const int* cu,
+                  const int* resume, int64_t M, int64_t B, int64_t W, int64_t nb, int64_t taps, int64_t act, int64_t f32, void* stream);
+
 /* ---- latent attention --------------------------------------------------------------------------------------------------
  * evo_latent_prep: row m of q (pitch ldq) holds H heads of [dn | dr] and behind them the down-projection [R | dr].  Rotates the dr part of
  * every head in place (pairs (i, i + n_rot / 2), angle pos[m] * inv_freq[i]); c [M, R] = the norm of the R part times w; kr [M, dr] = the
@@ -419,13 +480,6 @@ int evo_lightning_recurrent(const void* z, int64_t ld, void* o, float* state, co
 int evo_latent_prep(void* q, int64_t ldq, void* c, void* kr, void* cache, const void* w, const float* inv_freq, const int64_t* pos,
                     const int* seq, const int* cu, int64_t M, int64_t H, int64_t dn, int64_t dr, int64_t R, int64_t n_rot, int64_t ring,
                     int64_t rs, float eps, int64_t f32, void* stream);
-/* Causal attention over a sliding window with one sink per head in the denominator: o_i = sum_j p_ij v_j over 0 <= i - j < window,
- * p = exp(scale q.k) / (exp(sink) + sum exp(scale q.k)).  Per head q = [dn | dr] (pitch ldq), k = [kn (dn) | kr (dr, shared)], v (dv);
- * kn and v rows have pitch ldkv, o is [Mq, H dv].  A sequence's queries are its LAST cu_q lengths of its cu_k keys.  dv <= 512.
- * mfma 0: the any-size kernel (also taken for fp32 and beyond 256 key or value dimensions). */
-int evo_window_attn(const void* q, int64_t ldq, const void* kn, const void* v, int64_t ldkv, const void* kr, void* o, const int* cu_q,
-                    const int* cu_k, const float* sink, int64_t B, int64_t H, int64_t dn, int64_t dr, int64_t dv, int64_t window, int64_t max_q,
-                    float scale, int64_t f32, int64_t mfma, void* stream);
 /* Decode, one query per sequence (row b, position pos[b], its token already in the cache), in three launches:
  *   out [B, H, rs] = [W_uk,h^T q | rotated q | zeros];  n_split partial softmax sums over the ring (part_o [B, H, n_split, R] unnormalised,
  *   part_ml [B, H, n_split, 2] = running max in the log2 domain, denominator; mfma: 0 the any-size kernel, else the matrix cores with

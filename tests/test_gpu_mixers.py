@@ -112,7 +112,7 @@ def test_silu_gated_mlp(ops, M, I, K, grouped):
 @pytest.mark.parametrize("M,N,K,n", [(3, 70, 52, 33), (20, 512, 128, 256), (300, 512, 192, 256), (300, 512, 192, 512), (300, 512, 192, 200), (5129, 512, 128, 256)])
 def test_linear_with_silu_on_the_first_columns(ops, dt, M, N, K, n):
     x, w = rnd(M, K, seed=1, dt=dt), rnd(N, K, seed=2, dt=dt, scale=2.0 / math.sqrt(K))
-    got = ops.linear_silu(x.to(DEV), w.to(DEV), n)
+    got = ops.linear_act(x.to(DEV), w.to(DEV), "silu", n)
     want = x.double() @ w.double().T
     want[:, :n] = V.silu(want[:, :n])
     assert rel_err(got, want) < tol(dt, 8e-3, 5e-6)
