@@ -359,24 +359,33 @@ extern "C" int evo_window_attn(const void* q, int64_t ldq, const void* kn, const
     if (!f32 && mfma && dq <= (maps == 2 ? 128 : 256) && dv <= 256) {
         const bool vec = dn % 8 == 0 && dr % 8 == 0 && dv % 8 == 0 && ldq % 8 == 0 && ldkv % 8 == 0 &&
                          (((uintptr_t)q | (uintptr_t)kn | (uintptr_t)v | (uintptr_t)kr) & 15) == 0;
-#define WA(KS, DVB, QC, VEC, MAPS, MINW)                                                                                   \
+#define WA1(KS, DVB, QC, VEC, KEEP, MAPS, MINW)                                                                            \
     do {                                                                                                                   \
         a.n_qb = (int)((max_q + 64 * QC / MAPS - 1) / (64 * QC / MAPS));                                                   \
         const int64_t items = (int64_t)a.n_qb * H * B;                                                                     \
         if (items > 0x7ffffff0) return -1;                                                                                 \
-        const dim3 grid((unsigned)((items + 7) / 8 * 8));                                                                  \
-        if (kp) hipLaunchKernelGGL((window_attn_kernel<KS, DVB, QC, VEC, true, MAPS, MINW>), grid, dim3(256), 0, s, a, (int)B);   \
-        else hipLaunchKernelGGL((window_attn_kernel<KS, DVB, QC, VEC, false, MAPS, MINW>), grid, dim3(256), 0, s, a, (int)B);     \
+        hipLaunchKernelGGL((window_attn_kernel<KS, DVB, QC, VEC, KEEP, MAPS, MINW>), dim3((unsigned)((items + 7) / 8 * 8)), dim3(256), 0, s, a, (int)B); \
     } while (0)
+#define WA(KS, DVB, QC, VEC, MAPS, MINW) do { if (kp) WA1(KS, DVB, QC, VEC, true, MAPS, MINW); else WA1(KS, DVB, QC, VEC, false, MAPS, MINW); } while (0)
 #define WAV(KS, QC) do { if (dv <= 64) WA(KS, 4, QC, true, 1, 2); else if (dv <= 128) WA(KS, 8, QC, true, 1, 2); else WA(KS, 16, 1, true, 1, 2); } while (0)
 #define WA2(KS) do { if (dv <= 64) WA(KS, 4, 2, true, 2, 2); else if (dv <= 128) WA(KS, 8, 2, true, 2, 2); else WA(KS, 16, 2, true, 2, 1); } while (0)
         if (maps == 2) { if (!vec) WA(4, 16, 2, false, 2, 1); else if (dq <= 64) WA2(2); else WA2(4); }
         else if (!vec) { if (dq <= 64 && dv <= 64) WA(2, 4, 2, false, 1, 2); else WA(8, 16, 1, false, 1, 2); }
-        else if (dq <= 64) WAV(2, 2); else if (dq <= 128) WAV(4, 2); else if (dq <= 192) { if (kp) WAV(6, 1); else WAV(6, 2); }
-        else if (dv <= 128) WAV(8, 1); else WA(8, 16, 1, true, 1, 1);
+        else if (dq <= 64) WAV(2, 2);
+        else if (dq <= 128) WAV(4, 2);
+        else if (dq <= 192) {                                    // (kept tokens cost registers: one column block)
+            if (dv <= 64) WA(6, 4, 2, true, 1, 2);
+            else if (dv > 128) WA(6, 16, 1, true, 1, 2);
+            else if (kp) WA1(6, 8, 1, true, true, 1, 2);
+            else WA1(6, 8, 2, true, false, 1, 2);
+        }
+        else if (dv <= 64) WA(8, 4, 1, true, 1, 2);
+        else if (dv <= 128) WA(8, 8, 1, true, 1, 2);
+        else WA(8, 16, 1, true, 1, 1);
 #undef WA2
 #undef WAV
 #undef WA
+#undef WA1
         return evo_launch_status();
     }
     const dim3 grid((unsigned)max_q, (unsigned)H, (unsigned)B);

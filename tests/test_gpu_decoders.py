@@ -1,4 +1,5 @@
-"""GPU: whole Vozalorn models through the framework's entry points, against the plain fp64 reference run one sequence at a time."""
+"""GPU: whole models of the config.json families through the framework's entry points, against the plain fp64 references run one sequence at a
+time.  A case is "family/configuration"."""
 import json
 import os
 import subprocess
@@ -9,8 +10,13 @@ import pytest
 import torch
 from safetensors.torch import save_file
 
+import batodra_util
+import vozalorn_util
 import vozalorn_util as U
 
+FAMILIES = {"vozalorn": vozalorn_util, "batodra": batodra_util}
+ALL = [f"{f}/{n}" for f, u in FAMILIES.items() for n in sorted(u.CONFIGS)]
+EACH = pytest.mark.parametrize("family", sorted(FAMILIES))
 pytestmark = pytest.mark.gpu
 DEV = "cuda:0"
 DTYPES = pytest.mark.parametrize("dt", [torch.float32, torch.bfloat16], ids=["f32", "bf16"])
@@ -19,14 +25,20 @@ DTYPES = pytest.mark.parametrize("dt", [torch.float32, torch.bfloat16], ids=["f3
 NOISE = {}
 
 
+def parts(name):
+    u = FAMILIES[name.split("/")[0]]
+    cfg = u.CONFIGS[name.split("/")[1]]
+    return u, cfg, u.weights(cfg)
+
+
 def tol(name, dt):
     """fp32: rounding of fp32 sums; bf16: three times the worst row that rounding alone gives (U.rounding_noise)"""
     if dt == torch.float32:
         return 2e-4
     if name not in NOISE:
-        cfg = U.CONFIGS[name]
-        w, ids = U.weights(cfg), U.tokens(cfg, 200)
-        NOISE[name] = U.rounding_noise(cfg, w, ids, U.reference(cfg, w)(ids))
+        u, cfg, w = parts(name)
+        ids = U.tokens(cfg, 200)
+        NOISE[name] = U.rounding_noise(cfg, w, ids, u.reference(cfg, w)(ids))
     return 3 * NOISE[name][0]
 
 
@@ -36,9 +48,8 @@ def cases():
 
     def get(name, dt):
         if (name, dt) not in built:
-            cfg = U.CONFIGS[name]
-            w = U.weights(cfg)
-            built[name, dt] = (cfg, U.build(cfg, w, dtype=dt, device=DEV), U.reference(cfg, w))
+            u, cfg, w = parts(name)
+            built[name, dt] = (cfg, U.build(cfg, w, dtype=dt, device=DEV), u.reference(cfg, w))
         return built[name, dt]
     return get
 
@@ -50,7 +61,7 @@ def pool_of(m, n_slots, **kw):
 
 
 @DTYPES
-@pytest.mark.parametrize("name", sorted(U.CONFIGS))
+@pytest.mark.parametrize("name", ALL)
 def test_prompt_then_long_decoding(cases, name, dt):
     """A prompt in one pass, then 110 tokens one by one (every window of the configurations passes over decoded tokens); with the
     captured step where the dense shapes allow it."""
@@ -71,14 +82,15 @@ def test_prompt_then_long_decoding(cases, name, dt):
     if dt == torch.bfloat16:                                      # on average no worse than one rounding per op
         assert float(err.mean()) < 1.5 * NOISE[name][1]
     assert m.decode_graph and (m.decode_graph_replays == N - 1) == m._graph_shapes_ok(1)
-    if dt == torch.bfloat16 and name != "odd":
+    if dt == torch.bfloat16 and not name.endswith("/odd"):
         assert m._graph_shapes_ok(1)
 
 
 @DTYPES
 @pytest.mark.parametrize("cuts", [[2] * 40, [64, 16], [1, 79], [79, 1], [33, 2, 45]])
-def test_portions(cases, cuts, dt):
-    for name in ("order", "window_64"):
+@EACH
+def test_portions(cases, family, cuts, dt):
+    for name in (family + "/order", family + "/window_64"):
         cfg, m, ref = cases(name, dt)
         ids = U.tokens(cfg, 80)
         ipd = m.initialize_inference_params()
@@ -92,7 +104,8 @@ def test_portions(cases, cuts, dt):
 
 
 @DTYPES
-@pytest.mark.parametrize("name", ["plain", "odd", "wide_heads", "window_64"])
+@pytest.mark.parametrize("name", ["vozalorn/plain", "vozalorn/odd", "vozalorn/wide_heads", "vozalorn/window_64", "batodra/plain", "batodra/odd", "batodra/grouped",
+                                  "batodra/order", "batodra/window_64"])
 def test_unequal_requests_and_reused_slots(cases, name, dt):
     """Waves of unequal requests share a pool: packed prompts, pooled steps (captured), early ends, slots used again."""
     cfg, m, ref = cases(name, dt)
@@ -114,9 +127,10 @@ def test_unequal_requests_and_reused_slots(cases, name, dt):
             pool.release(s)
 
 
-def test_batch_does_not_change_a_request(cases):
+@EACH
+def test_batch_does_not_change_a_request(cases, family):
     """bf16: a prompt's logits alone and between others agree to rounding of the dense layers' different tilings."""
-    cfg, m, _ = cases("window_64", torch.bfloat16)
+    cfg, m, _ = cases(family + "/window_64", torch.bfloat16)
     a, others = U.tokens(cfg, 100, 1), [U.tokens(cfg, n, n) for n in (17, 400, 64)]
     with torch.inference_mode():
         alone = m.prefill_rows([torch.tensor(a).to(DEV)], [list(range(100))])[0][0]
@@ -124,11 +138,12 @@ def test_batch_does_not_change_a_request(cases):
     assert U.rel_err(mixed.float(), alone.float()) < 1.5e-2
 
 
-def test_long_prompt_in_segments(cases):
-    """Longer than a segment of the linear attention and than many window tiles; the last tokens against the reference."""
-    cfg, m, ref = cases("window_64", torch.bfloat16)
+@EACH
+def test_long_prompt_in_segments(cases, family):
+    """Longer than a segment of the recurrences and than many window tiles; the last tokens against the reference."""
+    cfg, m, ref = cases(family + "/window_64", torch.bfloat16)
     ids = U.tokens(cfg, 1500)
-    assert U.rel_err(m(torch.tensor([ids]).to(DEV))[0][0, -200:], ref(ids)[-200:]) < tol("window_64", torch.bfloat16)
+    assert U.rel_err(m(torch.tensor([ids]).to(DEV))[0][0, -200:], ref(ids)[-200:]) < tol(family + "/window_64", torch.bfloat16)
 
 
 def greedy(ref, ids, n):
@@ -138,9 +153,10 @@ def greedy(ref, ids, n):
     return ids[-n:]
 
 
-def test_greedy_generation(cases):
+@EACH
+def test_greedy_generation(cases, family):
     from evo_amd.generation import generate
-    cfg, m, ref = cases("plain", torch.float32)
+    cfg, m, ref = cases(family + "/plain", torch.float32)
     pool = pool_of(m, 2, top_k=1)
     prompts = ["ACGTAC", "GG", "TTTACGATCGATTA"]
     pool.generate(prompts, n_tokens=12, n_sample_per_prompt=2)
@@ -151,14 +167,15 @@ def test_greedy_generation(cases):
     assert out == [want, want]
 
 
-def test_bf16_generation_and_scoring_run(cases):
+@EACH
+def test_bf16_generation_and_scoring_run(cases, family):
     from evo_amd.scoring import score_sequences
-    cfg, m, ref = cases("window_64", torch.bfloat16)
+    cfg, m, ref = cases(family + "/window_64", torch.bfloat16)
     pool = pool_of(m, 3, top_k=1)
     pool.generate(["ACGTACGATTTA", "GG"], n_tokens=20)
     for row, lg, p in zip(pool.last_ids, pool.last_logits, ("ACGTACGATTTA", "GG")):
         want = ref(list(p.encode()) + row.tolist())[len(p) - 1:-1]
-        assert U.rel_err(lg, want) < tol("window_64", torch.bfloat16)
+        assert U.rel_err(lg, want) < tol(family + "/window_64", torch.bfloat16)
     got = score_sequences(["ACGTTA", "GGC"], m, pool.tok, device=DEV)
     for s, g in zip(["ACGTTA", "GGC"], got):
         ids = [0] + list(s.encode())
@@ -166,22 +183,69 @@ def test_bf16_generation_and_scoring_run(cases):
         assert abs(g - want) < 2e-2 * abs(want)
 
 
-def test_bad_ids_raise(cases):
-    cfg, m, _ = cases("plain", torch.bfloat16)
+@EACH
+def test_bad_ids_raise(cases, family):
+    cfg, m, _ = cases(family + "/plain", torch.bfloat16)
     with pytest.raises(IndexError):
         m(torch.tensor([[1, cfg["vocab"]]]).to(DEV))
 
 
-def test_command_line(tmp_path):
+@DTYPES
+@pytest.mark.parametrize("keep,window", [(0, 6), (3, 64), (70, 40), (65, 130)])
+def test_a_key_that_stands_out_at_every_distance(keep, window, dt):
+    """One token that takes most of the attention: inside and outside of the window, among the kept first tokens and just behind them, in
+    prompts and for decoded tokens."""
+    u = batodra_util
+    cfg = u.config([u.windowed(window=window, keep=keep, dim=32, rot=32, vdim=32)])
+    w = u.spiky(cfg, u.weights(cfg))
+    m, ref = U.build(cfg, w, dtype=dt, device=DEV), u.reference(cfg, w)
+    P, T = 2 * (keep + window) // 2 + 40, 2 * (keep + window) // 2 + 90
+    base = [t if t != 7 else 8 for t in U.tokens(cfg, T)]
+    noise = None
+    for at in sorted({0, 1, max(keep - 1, 0), keep, keep + 1, P - window, P - window + 1, P - 1, P - window + 20, T - window - 5}):
+        ids = base[:at] + [7] + base[at + 1:]
+        want = ref(ids)
+        if dt == torch.bfloat16 and noise is None:
+            noise = U.rounding_noise(cfg, w, ids, want)[0]
+        limit = 2e-4 if dt == torch.float32 else 3 * noise
+        assert U.rel_err(m(torch.tensor([ids]).to(DEV))[0][0], want) < limit
+        ipd = m.initialize_inference_params()
+        got = [m(torch.tensor([ids[:P]]).to(DEV), ipd)[0][0]]
+        for t in range(P, T):
+            ipd["mha"].seqlen_offset = ipd["hyena"].seqlen_offset = t
+            got.append(m(torch.tensor([ids[t:t + 1]]).to(DEV), ipd)[0][0])
+        m.release_decode_graph()
+        assert U.rel_err(torch.cat(got), want) < limit, at
+
+
+def test_caches_grow_under_the_captured_step(cases):
+    """Decoding beyond the room the prompt's caches were given: they are enlarged between replays, the step is captured again."""
+    cfg, m, ref = cases("batodra/window_64", torch.bfloat16)
+    ids = U.tokens(cfg, 120)
+    want = ref(ids)
+    spare, m.spare_positions = m.spare_positions, 8
+    try:
+        ipd = m.initialize_inference_params()
+        got = [m(torch.tensor([ids[:20]]).to(DEV), ipd)[0][0]]
+        for t in range(20, 120):
+            ipd["mha"].seqlen_offset = ipd["hyena"].seqlen_offset = t
+            got.append(m(torch.tensor([ids[t:t + 1]]).to(DEV), ipd)[0][0])
+    finally:
+        m.spare_positions = spare
+        m.release_decode_graph()
+    assert U.rel_err(torch.cat(got), want) < tol("batodra/window_64", torch.bfloat16)
+
+
+@EACH
+def test_command_line(tmp_path, family):
     """scripts/generate.py on a model folder, and a trace replayed by bin/trace_run."""
     root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
-    cfg = U.CONFIGS["plain"]
-    w = U.weights(cfg)
+    u, cfg, w = parts(family + "/plain")
     (tmp_path / "config.json").write_text(json.dumps(cfg))
     save_file(w, str(tmp_path / "model.safetensors"))
     out = subprocess.run([sys.executable, "-m", "scripts.generate", "--model-dir", str(tmp_path), "--dtype", "float32", "--prompt", "ACGT",
                           "--n-samples", "1", "--n-tokens", "6", "--top-k", "1", "--verbose", "0"], cwd=root, capture_output=True, text=True, timeout=120)
-    ref = U.reference(cfg, w)
+    ref = u.reference(cfg, w)
     from evo_amd.tokenizer import CharLevelTokenizer
     assert out.returncode == 0, out.stderr[-2000:]
     assert CharLevelTokenizer(cfg["vocab"]).detokenize(greedy(ref, b"ACGT", 6)) in out.stdout
@@ -195,4 +259,4 @@ def test_command_line(tmp_path):
     assert [l for l in run.stdout.splitlines() if l.startswith("done")] == [f"done {i}" for i in range(11)]
     want = ref(ids)
     got = [np.fromfile(tmp_path / f"{i}.f32", dtype="<f4").reshape(-1, cfg["vocab"]) for i in range(11)]
-    assert U.rel_err(np.concatenate(got), want[[3] + list(range(19, 30))]) < tol("plain", torch.bfloat16)
+    assert U.rel_err(np.concatenate(got), want[[3] + list(range(19, 30))]) < tol(family + "/plain", torch.bfloat16)
