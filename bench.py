@@ -546,12 +546,12 @@ def main():
     ap.add_argument("--skip-gen", action="store_true")
     ap.add_argument("--steps-131k", type=int, default=2)
     ap.add_argument("--sp-timeout", type=float, default=420.0, help="N > 1: seconds the sequence-parallel 131k leg may take")
-    ap.add_argument("--arch", default=None, choices=["vozalorn"], help="instead of the default workload: prefill and decode throughput of this "
-                    "architecture at 7B layer sizes beside a StripedHyena of the same width and depth (tools/bench_arch.py), one JSON line")
+    ap.add_argument("--arch", default=None, choices=["vozalorn", "batodra"], help="instead of the default workload: prefill and decode throughput "
+                    "of this architecture at 7B layer sizes beside the closest models of the same width and depth (tools/bench_arch.py), one JSON line")
     args = ap.parse_args()
     if args.arch:
         from tools.bench_arch import run
-        print(json.dumps(run("cuda:0", steps=args.steps)))
+        print(json.dumps(run("cuda:0", arch=args.arch, steps=args.steps)))
         return
 
     import torch.distributed as dist
