@@ -10,6 +10,8 @@
 // (1) every segment's decay product and end state from zero, (2) a scan over segments, (3) outputs.
 #include "mixers_common.h"
 #include "../../include/evo_mi355x.h"
+#include <cstdlib>
+#include <type_traits>
 
 #define LOG2E 1.4426950408889634f
 #define RT 64                                                    // tokens per tile
@@ -23,18 +25,38 @@ struct RgArgs {
     int W, nb, bs, taps, n_seg, seg_len, n_cg, act, rows;
 };
 
-__device__ __forceinline__ float rcp1p_exp2(float e) { return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(e)); }   // 1 / (1 + 2^e)
+typedef __bf16 rg_bf16x2 __attribute__((ext_vector_type(2)));
+__device__ __forceinline__ float dot2(uint32_t a, uint32_t b, float c) {
+    return __builtin_amdgcn_fdot2_f32_bf16(__builtin_bit_cast(rg_bf16x2, a), __builtin_bit_cast(rg_bf16x2, b), c, false);
+}
+// the values of a lane's neighbours in the four 16-lane rows of a wave: swap16 -> (even row of its pair, odd row), swap32 -> (lower half, upper half)
+__device__ __forceinline__ void swap16(float v, float& even, float& odd) {
+    const auto r = __builtin_amdgcn_permlane16_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+    even = __uint_as_float(r[0]); odd = __uint_as_float(r[1]);
+}
+__device__ __forceinline__ void swap32(float v, float& low, float& high) {
+    const auto r = __builtin_amdgcn_permlane32_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+    low = __uint_as_float(r[0]); high = __uint_as_float(r[1]);
+}
+// gates of one channel: decay a and input sqrt(1 - a^2) i u from the maps' results.  sqrt(x) / E = x rsqrt(x E^2); x is 0 (a = 1) or at least 2^-24.
+__device__ __forceinline__ void gate(float zr, float zi, float c2, float u, float& al, float& add) {
+    al = __builtin_amdgcn_exp2f(c2 * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-LOG2E * zr)));
+    const float x = fmaxf(fmaf(-al, al, 1.0f), 1e-30f), e = 1.0f + __builtin_amdgcn_exp2f(-LOG2E * zi);
+    add = x * __builtin_amdgcn_rsqf(x * e * e) * u;
+}
 
 // ------------------------------------------------------------------------------------------------ prompts
 // KS: 32-wide steps of a block, NW: waves.  OUT: outputs and the sequence's end state; otherwise a segment's (product of a, end state from zero).
 template <int KS, int NW, bool OUT>
 __global__ __launch_bounds__(64 * NW) void rglru_chunk_kernel(RgArgs a) {
-    constexpr int KP = 32 * KS, PR = KP + 8, NT = 64 * NW;
+    constexpr int KP = 32 * KS, PR = KP + 8, NT = 64 * NW, NC = 16 * NW, YP = NC + 8;
     constexpr int IT = (16 * 4 * KS + NT - 1) / NT;              // staged runs (four tokens x eight channels) per thread
     constexpr bool AHEAD = KS < 12;                              // the next tile's rows are requested a tile ahead (wide blocks: no registers left)
     extern __shared__ __attribute__((aligned(16))) uint16_t lds[];
     uint16_t* const tile = lds;                                  // [2][RT][PR]
-    float* const cw = (float*)(lds + 2 * RT * PR);               // [TAPS + 1][KP]: taps, oldest first, then the bias
+    uint32_t* const cw = (uint32_t*)(lds + 2 * RT * PR);         // [2][KP] taps as bf16 pairs, oldest first; [KP] the bias
+    float* const cb = (float*)(cw + 2 * KP);
+    uint16_t* const yo = (uint16_t*)(cb + KP);                   // [2][RT][YP] y, replaced by the outputs where they are made
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int c16 = lane & 15, g = lane >> 4;
     const int cg = blockIdx.x % a.n_cg, seg = blockIdx.x / a.n_cg, n = blockIdx.y, b = blockIdx.z;
@@ -47,15 +69,19 @@ __global__ __launch_bounds__(64 * NW) void rglru_chunk_kernel(RgArgs a) {
     const int ch = cg * 16 * NW + 16 * wave + c16, cc = ch < bs ? ch : bs - 1;   // this lane's channel of the block (clamped for loads)
     const int wch = n * bs + cc;                                 // ... of the whole width
     const uint16_t* zx = (const uint16_t*)a.z + (int64_t)row0 * a.ld + W + n * bs;
-    const uint16_t* zy = (const uint16_t*)a.z + (int64_t)row0 * a.ld + wch;
+    const uint16_t* zy = (const uint16_t*)a.z + (int64_t)row0 * a.ld + n * bs;
     float* st = a.state ? a.state + (int64_t)b * (1 + a.taps) * W + n * bs : nullptr;
 
     for (int i = tid; i < KP; i += NT) {                         // taps and bias of this block's channels
+        uint32_t w[TAPS];
+#pragma unroll
         for (int t = 0; t < TAPS; ++t) {
             const int k = t - (TAPS - a.taps);
-            cw[t * KP + i] = i < bs && k >= 0 ? ld1((const uint16_t*)a.conv + (int64_t)(n * bs + i) * a.taps + k) : 0.f;
+            w[t] = i < bs && k >= 0 ? ((const uint16_t*)a.conv)[(int64_t)(n * bs + i) * a.taps + k] : 0u;
         }
-        cw[TAPS * KP + i] = i < bs ? ld1((const uint16_t*)a.conv_b + n * bs + i) : 0.f;
+        cw[i] = w[0] | w[1] << 16;
+        cw[KP + i] = w[2] | w[3] << 16;
+        cb[i] = i < bs ? ld1((const uint16_t*)a.conv_b + n * bs + i) : 0.f;
     }
     for (int i = tid; i < 2 * RT * (PR - bs); i += NT) tile[i / (PR - bs) * PR + bs + i % (PR - bs)] = 0;   // columns behind the block
     mx_frag wr[KS], wi[KS];                                      // rows of the gate maps: this lane's channel
@@ -71,15 +97,18 @@ __global__ __launch_bounds__(64 * NW) void rglru_chunk_kernel(RgArgs a) {
     // staged run: tokens 4 q .. 4 q + 3, channels 8 d .. 8 d + 7 of the block
     const int nd = bs / 8;
     mx_u32x4 xr[AHEAD ? IT : 1][TAPS + 3];
-    auto load_run = [&](int t0, int i, mx_u32x4* x) __attribute__((always_inline)) {
+    const uint32_t row_bytes = (uint32_t)a.ld * 2;
+    auto load_run = [&](int t0, int i, mx_u32x4* x) __attribute__((always_inline)) {   // (uniform base, 32-bit offsets: rows t0 - 3 + 4 q + u, clamped)
         int it = tid + NT * i;
         it = it < 16 * nd ? it : 16 * nd - 1;
-        const int q = it / nd, d = it - q * nd;
+        const int q = it / nd, d = it - q * nd, tb = t0 < len_all ? t0 : len_all - 1;
+        const int lo = tb < TAPS - 1 ? TAPS - 1 - tb : 0, hi = len_all - 1 - tb + TAPS - 1;
+        const char* base = (const char*)(zx + (int64_t)(tb - (TAPS - 1)) * a.ld);
 #pragma unroll
         for (int u = 0; u < TAPS + 3; ++u) {
-            int t = t0 + 4 * q + u - (TAPS - 1);
-            t = t < 0 ? 0 : (t < len_all ? t : len_all - 1);
-            x[u] = *(const mx_u32x4*)(zx + t * a.ld + 8 * d);
+            int r = 4 * q + u;
+            r = r < lo ? lo : (r < hi ? r : hi);
+            x[u] = *(const mx_u32x4*)(base + (uint32_t)((uint32_t)r * row_bytes + 16u * (uint32_t)d));
         }
     };
     auto load_x = [&](int t0) __attribute__((always_inline)) {
@@ -93,41 +122,28 @@ __global__ __launch_bounds__(64 * NW) void rglru_chunk_kernel(RgArgs a) {
             if (!AHEAD) load_run(t0, i, xr[0]);
             if (it >= 16 * nd) break;
             const int q = it / nd, d = it - q * nd;
-            float acc[4][8];
-            {
-                const float4 p = *(const float4*)(cw + TAPS * KP + 8 * d), r = *(const float4*)(cw + TAPS * KP + 8 * d + 4);
+            if (t0 == 0 && q == 0) {                             // before this portion: the cached inputs, zeros before the sequence
 #pragma unroll
-                for (int v = 0; v < 4; ++v) {
-                    acc[v][0] = p.x; acc[v][1] = p.y; acc[v][2] = p.z; acc[v][3] = p.w;
-                    acc[v][4] = r.x; acc[v][5] = r.y; acc[v][6] = r.z; acc[v][7] = r.w;
-                }
-            }
-            float w[TAPS][8];
-#pragma unroll
-            for (int t = 0; t < TAPS; ++t) {
-                const float4 p = *(const float4*)(cw + t * KP + 8 * d), r = *(const float4*)(cw + t * KP + 8 * d + 4);
-                w[t][0] = p.x; w[t][1] = p.y; w[t][2] = p.z; w[t][3] = p.w; w[t][4] = r.x; w[t][5] = r.y; w[t][6] = r.z; w[t][7] = r.w;
-            }
-#pragma unroll
-            for (int u = 0; u < TAPS + 3; ++u) {
-                float x[8];
-#pragma unroll
-                for (int e = 0; e < 4; ++e) { x[2 * e] = bf_lo(xr[xi][u][e]); x[2 * e + 1] = bf_hi(xr[xi][u][e]); }
-                if (t0 == 0 && 4 * q + u < TAPS - 1) {           // before this portion: the cached inputs, zeros before the sequence
-                    const int back = TAPS - 1 - 4 * q - u;       // tokens before the portion's first, 1 .. TAPS - 1
+                for (int u = 0; u < TAPS - 1; ++u) {
+                    const int back = TAPS - 1 - u;               // tokens before the portion's first
                     const int64_t p = a.pos[row0] - back;
                     const bool have = go_on && p >= 0 && back < a.taps;
-                    const float* h = st + (1 + (have ? (int)(p % a.taps) : 0)) * (int64_t)W + 8 * d;
-#pragma unroll
-                    for (int e = 0; e < 8; ++e) x[e] = have ? h[e] : 0.f;
+                    float h[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+                    if (have) vec_io<float, 8>::load(st + (1 + (int)(p % a.taps)) * (int64_t)W + 8 * d, h);
+                    xr[xi][u] = mx_u32x4{pack_bf2(h[0], h[1]), pack_bf2(h[2], h[3]), pack_bf2(h[4], h[5]), pack_bf2(h[6], h[7])};
                 }
+            }
+            // two taps per instruction: operands are pairs of adjacent tokens of one channel
+            float acc[4][8];
 #pragma unroll
-                for (int v = 0; v < 4; ++v) {
-                    const int t = u - v;                         // tap of input u for token v
-                    if (t < 0 || t >= TAPS) continue;
+            for (int e = 0; e < 8; ++e) {
+                const uint32_t w0 = cw[8 * d + e], w1 = cw[KP + 8 * d + e], pick = e & 1 ? 0x07060302u : 0x05040100u;
+                const float c = cb[8 * d + e];
+                uint32_t pr[TAPS + 3];
 #pragma unroll
-                    for (int e = 0; e < 8; ++e) acc[v][e] = fmaf(w[t][e], x[e], acc[v][e]);
-                }
+                for (int u = 1; u < TAPS + 3; ++u) pr[u] = __builtin_amdgcn_perm(xr[xi][u][e >> 1], xr[xi][u - 1][e >> 1], pick);
+#pragma unroll
+                for (int v = 0; v < 4; ++v) acc[v][e] = dot2(pr[v + 3], w1, dot2(pr[v + 1], w0, c));
             }
 #pragma unroll
             for (int v = 0; v < 4; ++v)
@@ -141,63 +157,101 @@ __global__ __launch_bounds__(64 * NW) void rglru_chunk_kernel(RgArgs a) {
         if (a.seg && (seg > 0 || go_on)) S = a.seg[(((int64_t)b * a.n_seg + seg) * 2 + 1) * W + wch];
         else if (go_on) S = st[cc];
     }
+    // y and the outputs move 16 bytes at a time: thread (row, run of eight channels) of two runs, the same ones in both directions
+    mx_u32x4 yv[2];
+    auto load_y = [&](int t0) __attribute__((always_inline)) {
+        if (!OUT) return;
+        const int tb = t0 < s_hi ? t0 : s_hi - 1;
+        const char* base = (const char*)(zy + (int64_t)tb * a.ld);
+#pragma unroll
+        for (int k = 0; k < 2; ++k) {
+            const int it = tid + NT * k, r = it / (NC / 8), c = cg * NC + 8 * (it % (NC / 8));
+            yv[k] = *(const mx_u32x4*)(base + (uint32_t)((uint32_t)(r < s_hi - tb ? r : s_hi - 1 - tb) * row_bytes + 2u * (uint32_t)(c < bs ? c : bs - 8)));
+        }
+    };
+    auto store_o = [&](int t0, const uint16_t* src) __attribute__((always_inline)) {
+        char* base = (char*)((uint16_t*)a.o + ((int64_t)row0 + t0) * W + n * bs);
+#pragma unroll
+        for (int k = 0; k < 2; ++k) {
+            const int it = tid + NT * k, r = it / (NC / 8), j = it % (NC / 8), c = cg * NC + 8 * j;
+            const uint4 v = *(const uint4*)(src + r * YP + 8 * j);
+            if (t0 + r < s_hi && c < bs) *(uint4*)(base + (uint32_t)((uint32_t)r * (uint32_t)W * 2u + 2u * (uint32_t)c)) = v;
+        }
+    };
     load_x(s_lo);
+    load_y(s_lo);
     __syncthreads();                                             // (taps)
     int buf = 0;
     for (int t0 = s_lo; t0 < s_hi; t0 += RT, buf ^= 1) {
         uint16_t* const ut = tile + buf * RT * PR;
+        uint16_t* const yt = yo + buf * RT * YP;
         convolve(t0, ut);
-        __syncthreads();                                         // (the other buffer's readers are past this tile's barrier as well)
-        load_x(t0 + RT);                                         // (past the end: valid rows again, not used)
-        uint16_t yv[16];
         if (OUT) {
 #pragma unroll
-            for (int k = 0; k < 16; ++k) {
-                const int t = t0 + 16 * (k >> 2) + 4 * g + (k & 3);
-                yv[k] = zy[(int64_t)(t < s_hi ? t : s_hi - 1) * a.ld];
+            for (int k = 0; k < 2; ++k) {
+                const int it = tid + NT * k;
+                *(mx_u32x4*)(yt + it / (NC / 8) * YP + 8 * (it % (NC / 8))) = yv[k];
             }
         }
+        __syncthreads();                                         // (the other buffers' readers are past this tile's barrier as well)
+        load_x(t0 + RT);                                         // (past the end: valid rows again, not used)
+        load_y(t0 + RT);
+        if (OUT && t0 > s_lo) store_o(t0 - RT, yo + (buf ^ 1) * RT * YP);
         __builtin_amdgcn_sched_barrier(0);
-        const bool full = t0 + RT <= s_hi;
-#pragma unroll
-        for (int tb = 0; tb < 4; ++tb) {
-            f32x4_t zr = {br, br, br, br}, zi = {bi, bi, bi, bi};
+        // the gate maps of a 16-token block run ahead of the arithmetic on the one before
+        f32x4_t zr[2], zi[2];
+        auto maps = [&](int tb) __attribute__((always_inline)) {
+            f32x4_t r = {br, br, br, br}, i = {bi, bi, bi, bi};
 #pragma unroll
             for (int ks = 0; ks < KS; ++ks) {
                 const mx_frag uf = __builtin_bit_cast(mx_frag, *(const uint4*)(ut + (16 * tb + c16) * PR + 32 * ks + 8 * g));
-                zr = mfma16(uf, wr[ks], zr);
-                zi = mfma16(uf, wi[ks], zi);
+                r = mfma16(uf, wr[ks], r);
+                i = mfma16(uf, wi[ks], i);
             }
+            zr[tb & 1] = r;
+            zi[tb & 1] = i;
+        };
+        auto walk = [&](auto full) __attribute__((always_inline)) {
+#pragma unroll
+        for (int tb = 0; tb < 4; ++tb) {
+            if (tb < 3) maps(tb + 1);
             float pa[4], ps[4];                                  // running (product of a, state from zero) over this lane's four tokens
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const float u = bf_to_f(ut[(16 * tb + 4 * g + r) * PR + cc]);
-                float al = __builtin_amdgcn_exp2f(c2 * rcp1p_exp2(-LOG2E * zr[r]));
-                float add = __builtin_amdgcn_sqrtf(fmaxf(fmaf(-al, al, 1.0f), 0.f)) * rcp1p_exp2(-LOG2E * zi[r]) * u;
-                if (!full && t0 + 16 * tb + 4 * g + r >= s_hi) { al = 1.f; add = 0.f; }   // past the end: the state stays
+                float al, add;
+                gate(zr[tb & 1][r], zi[tb & 1][r], c2, u, al, add);
+                if (!decltype(full)::value && t0 + 16 * tb + 4 * g + r >= s_hi) { al = 1.f; add = 0.f; }   // past the end: the state stays
                 pa[r] = r ? pa[r - 1] * al : al;
                 ps[r] = r ? fmaf(ps[r - 1], al, add) : add;
             }
-            // inclusive scan over the four lane groups, then this group's incoming state
-            float ga = pa[3], gs = ps[3];
-            float ua = __shfl_up(ga, 16, 64), us = __shfl_up(gs, 16, 64);
-            if (g >= 1) { gs = fmaf(us, ga, gs); ga *= ua; }
-            ua = __shfl_up(ga, 32, 64); us = __shfl_up(gs, 32, 64);
-            if (g >= 2) { gs = fmaf(us, ga, gs); ga *= ua; }
-            const float end = fmaf(ga, S, gs);                   // state behind this group's tokens
-            float in = __shfl_up(end, 16, 64);
-            if (g == 0) in = S;
-            if (!OUT) A *= __shfl(ga, 48 + c16, 64);
-            S = __shfl(end, 48 + c16, 64);
+            // composition over the four lane groups: every lane gets the even and odd member of its pair of groups, then both pairs
+            float ea, oa, es, os, la, ha, ls, hs;
+            swap16(pa[3], ea, oa);
+            swap16(ps[3], es, os);
+            swap32(ea * oa, la, ha);
+            swap32(fmaf(es, oa, os), ls, hs);
+            const float mid = fmaf(la, S, ls);                   // state behind the lower two groups
+            float in = g >= 2 ? mid : S;
+            if (g & 1) in = fmaf(ea, in, es);
+            if (!OUT) A *= la * ha;
+            S = fmaf(ha, mid, hs);
             if (OUT) {
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {
-                    const int t = t0 + 16 * tb + 4 * g + r;
-                    const float v = fmaf(pa[r], in, ps[r]) * bf_to_f(yv[4 * tb + r]);
-                    if (t < s_hi && ch < bs) ((uint16_t*)a.o)[((int64_t)row0 + t) * W + wch] = f_to_bf(v);
+                    uint16_t* e = yt + (16 * tb + 4 * g + r) * YP + 16 * wave + c16;
+                    *e = f_to_bf(fmaf(pa[r], in, ps[r]) * bf_to_f(*e));
                 }
             }
         }
+        };
+        maps(0);
+        if (t0 + RT <= s_hi) walk(std::true_type());
+        else walk(std::false_type());
+    }
+    if (OUT) {
+        __syncthreads();
+        store_o((s_hi - 1 - s_lo) / RT * RT + s_lo, yo + (buf ^ 1) * RT * YP);
     }
     if (g == 0 && ch < bs) {
         if (!OUT) {
@@ -245,7 +299,7 @@ extern "C" int evo_rglru_chunk_bf16(const void* z, int64_t ld, void* o, float* s
     if (!rg_sizes(z, o, conv, conv_b, ra, ra_b, ri, ri_b, decay, pos, ld, B, W, nb, taps) || !cu || (resume && !state)) return -1;
     const int64_t bs = W / nb;
     if (bs % 8 || bs > 384 || taps > TAPS || max_len <= 0 || max_len > 0x3fffffff || seg_len <= 0 || seg_len % RT || ld % 8) return -1;
-    if (((uintptr_t)z | (uintptr_t)ra | (uintptr_t)ri) & 15) return -1;
+    if ((((uintptr_t)z | (uintptr_t)ra | (uintptr_t)ri | (uintptr_t)o | (uintptr_t)state) & 15) || ld > 0xffffff || W > 0xffffff) return -1;
     const int64_t n_seg = (max_len + seg_len - 1) / seg_len;
     if (n_seg > 1 && !seg) return -1;
     const int nw = bs <= 64 ? 4 : 8;
@@ -257,7 +311,7 @@ extern "C" int evo_rglru_chunk_bf16(const void* z, int64_t ld, void* o, float* s
     const dim3 grid((unsigned)(n_seg * n_cg), (unsigned)nb, (unsigned)B);
 #define RC(KS, NW)                                                                                                         \
     do {                                                                                                                   \
-        constexpr int bytes = 2 * RT * (32 * KS + 8) * 2 + (TAPS + 1) * 32 * KS * 4;                                       \
+        constexpr int bytes = 2 * RT * (32 * KS + 8) * 2 + 3 * 32 * KS * 4 + 2 * RT * (16 * NW + 8) * 2;                                       \
         if (bytes > 64 * 1024) {                                                                                           \
             (void)hipFuncSetAttribute((const void*)rglru_chunk_kernel<KS, NW, false>, hipFuncAttributeMaxDynamicSharedMemorySize, bytes); \
             (void)hipFuncSetAttribute((const void*)rglru_chunk_kernel<KS, NW, true>, hipFuncAttributeMaxDynamicSharedMemorySize, bytes);  \
@@ -275,79 +329,103 @@ extern "C" int evo_rglru_chunk_bf16(const void* z, int64_t ld, void* o, float* s
 }
 
 // ------------------------------------------------------------------------------------------------ decode
-// One token per sequence.  A workgroup: 16 channels of one block for up to 16 sequences; the block's convolution outputs are rebuilt in LDS (a
-// few KB from L2), the four waves are the two gate maps x the halves of the sum, a thread ends with one channel of one sequence.
-template <int KS>
-__global__ __launch_bounds__(256) void rglru_step_kernel(RgArgs a) {
-    constexpr int KP = 32 * KS, PR = KP + 8, KH = (KS + 1) / 2;
+// One token per sequence.  A workgroup: 16 CG channels of one block for up to 16 sequences; the block's convolution outputs are rebuilt in LDS (a
+// few KB from L2), a wave is one of the two gate maps, one half of its sum and 16 of the channels, a thread ends with one channel of one
+// sequence.  The rows of a ring are requested before the position is known: which tap a row meets is settled afterwards.
+template <int KS, int CG>
+__global__ __launch_bounds__(256 * CG) void rglru_step_kernel(RgArgs a) {
+    constexpr int KP = 32 * KS, PR = KP + 8, KH = (KS + 1) / 2, NT = 256 * CG, NC = 16 * CG;
     __shared__ __attribute__((aligned(16))) uint16_t ut[16 * PR];
-    __shared__ float part[4][16][17];
+    __shared__ __attribute__((aligned(16))) float cw[(TAPS + 1) * KP];   // taps, oldest first, then a row of zeros
+    __shared__ float part[2][2][16][NC + 1];
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int c16 = lane & 15, g = lane >> 4;
-    const int n = blockIdx.y, b0 = blockIdx.z * 16, bs = a.bs, W = a.W, rows = a.rows - b0 < 16 ? a.rows - b0 : 16;
-    const int c0 = blockIdx.x * 16, gate = wave & 1, ks0 = (wave >> 1) * KH;
+    const int n = blockIdx.y, b0 = blockIdx.z * 16, bs = a.bs, W = a.W, taps = a.taps, rows = a.rows - b0 < 16 ? a.rows - b0 : 16;
+    const int c0 = blockIdx.x * NC, map = wave & 1, half = (wave >> 1) & 1, cg = wave >> 2;
     mx_frag wf[KH];
     {
-        const uint16_t* w = (const uint16_t*)(gate ? a.ri : a.ra) + ((int64_t)n * bs + (c0 + c16 < bs ? c0 + c16 : bs - 1)) * bs;
+        const int c = c0 + 16 * cg + c16;
+        const uint16_t* w = (const uint16_t*)(map ? a.ri : a.ra) + ((int64_t)n * bs + (c < bs ? c : bs - 1)) * bs;
 #pragma unroll
         for (int i = 0; i < KH; ++i) {
-            const int k = 32 * (ks0 + i) + 8 * g;
+            const int k = 32 * (half * KH + i) + 8 * g;
             wf[i] = __builtin_bit_cast(mx_frag, *(const mx_u32x4*)(w + (k < bs ? k : bs - 8)));
         }
     }
     const uint16_t* z = (const uint16_t*)a.z;
-    const int nd = KP / 8;
-    for (int it = tid; it < 16 * nd; it += 256) {                // eight channels of one sequence
-        const int i = it / nd, d = 8 * (it - i * nd);
-        uint4 u = make_uint4(0u, 0u, 0u, 0u);
-        if (i < rows && d < bs) {
-            const int b = b0 + i;
-            const int64_t p = a.pos[b];
-            float x[8], acc[8];
-            vec_io<uint16_t, 8>::load(z + b * a.ld + W + n * bs + d, x);
-            if (a.in_b) {
-                float ib[8];
-                vec_io<uint16_t, 8>::load((const uint16_t*)a.in_b + W + n * bs + d, ib);
+    // what this thread's channel of this thread's sequence needs at the end
+    const int mi = tid / NC, mc = c0 + tid % NC, wc = n * bs + (mc < bs ? mc : bs - 1), mb = b0 + (mi < rows ? mi : rows - 1);
+    float* st = a.state + (int64_t)mb * (1 + taps) * W + wc;
+    const float S0 = st[0], dec = a.decay[wc] * LOG2E, br = ld1((const uint16_t*)a.ra_b + wc), bi = ld1((const uint16_t*)a.ri_b + wc);
+    float mx = ld1(z + mb * a.ld + W + wc), my = ld1(z + mb * a.ld + wc);
+    if (a.in_b) { mx += ld1((const uint16_t*)a.in_b + W + wc); my += ld1((const uint16_t*)a.in_b + wc); }
+    const int64_t mpos = a.pos[mb];
+
+    for (int i = tid; i < (taps + 1) * KP; i += NT) {
+        const int t = i / KP, c = i - t * KP;
+        cw[i] = t < taps && c < bs ? ld1((const uint16_t*)a.conv + (int64_t)(n * bs + c) * taps + t) : 0.f;
+    }
+    constexpr int ND = KP / 8, IT = (16 * ND + NT - 1) / NT;     // runs of eight channels of one sequence, per thread
+    float acc[IT][8], h[IT][TAPS][8], x[IT][8];
 #pragma unroll
-                for (int e = 0; e < 8; ++e) x[e] += ib[e];
-            }
-            const uint16_t* cw = (const uint16_t*)a.conv + (int64_t)(n * bs + d) * a.taps;
-            vec_io<uint16_t, 8>::load((const uint16_t*)a.conv_b + n * bs + d, acc);
+    for (int k = 0; k < IT; ++k) {
+        const int it = tid + NT * k, i = it / ND, d = 8 * (it % ND), b = b0 + (i < rows ? i : rows - 1), dc = d < bs ? d : 0;
+        vec_io<uint16_t, 8>::load(z + b * a.ld + W + n * bs + dc, x[k]);
+        vec_io<uint16_t, 8>::load((const uint16_t*)a.conv_b + n * bs + dc, acc[k]);
 #pragma unroll
-            for (int e = 0; e < 8; ++e) acc[e] = fmaf(ld1(cw + e * a.taps + a.taps - 1), x[e], acc[e]);
-            for (int back = 1; back < a.taps; ++back) {
-                if (p - back < 0) break;
-                float h[8];
-                vec_io<float, 8>::load(a.state + ((int64_t)b * (1 + a.taps) + 1 + (p - back) % a.taps) * W + n * bs + d, h);
+        for (int t = 0; t < TAPS; ++t)                           // (fewer taps: the last row again, with weight zero)
+            vec_io<float, 8>::load(a.state + ((int64_t)b * (1 + taps) + 1 + (t < taps ? t : taps - 1)) * W + n * bs + dc, h[k][t]);
+        if (a.in_b) {
+            float ib[8];
+            vec_io<uint16_t, 8>::load((const uint16_t*)a.in_b + W + n * bs + dc, ib);
 #pragma unroll
-                for (int e = 0; e < 8; ++e) acc[e] = fmaf(ld1(cw + e * a.taps + a.taps - 1 - back), h[e], acc[e]);
-            }
-            u = make_uint4(pack_bf2(acc[0], acc[1]), pack_bf2(acc[2], acc[3]), pack_bf2(acc[4], acc[5]), pack_bf2(acc[6], acc[7]));
+            for (int e = 0; e < 8; ++e) x[k][e] += ib[e];
         }
-        *(uint4*)(ut + i * PR + d) = u;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int k = 0; k < IT; ++k) {
+        const int it = tid + NT * k, i = it / ND, d = 8 * (it % ND);
+        if (it >= 16 * ND) break;
+        const int64_t p = a.pos[b0 + (i < rows ? i : rows - 1)];
+        const int cur = (int)(p % taps);
+        auto add = [&](int row, const float* v) {
+            float w[8];
+            vec_io<float, 8>::load(cw + row * KP + d, w);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) acc[k][e] = fmaf(w[e], v[e], acc[k][e]);
+        };
+        add(taps - 1, x[k]);
+#pragma unroll
+        for (int t = 0; t < TAPS; ++t) {
+            const int back = cur - t + (cur < t ? taps : 0);     // tokens between this one and the row's
+            const bool have = t < taps && back > 0 && p - back >= 0;
+            float v[8];
+#pragma unroll
+            for (int e = 0; e < 8; ++e) v[e] = have ? h[k][t][e] : 0.f;
+            add(have ? taps - 1 - back : taps, v);
+        }
+        const bool on = i < rows && d < bs;
+        *(uint4*)(ut + i * PR + d) = make_uint4(on ? pack_bf2(acc[k][0], acc[k][1]) : 0u, on ? pack_bf2(acc[k][2], acc[k][3]) : 0u,
+                                                on ? pack_bf2(acc[k][4], acc[k][5]) : 0u, on ? pack_bf2(acc[k][6], acc[k][7]) : 0u);
     }
     __syncthreads();
     f32x4_t s = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int i = 0; i < KH; ++i)
-        if (ks0 + i < KS) s = mfma16(__builtin_bit_cast(mx_frag, *(const uint4*)(ut + c16 * PR + 32 * (ks0 + i) + 8 * g)), wf[i], s);
+        if (half * KH + i < KS) s = mfma16(__builtin_bit_cast(mx_frag, *(const uint4*)(ut + c16 * PR + 32 * (half * KH + i) + 8 * g)), wf[i], s);
 #pragma unroll
-    for (int r = 0; r < 4; ++r) part[wave][4 * g + r][c16] = s[r];
+    for (int r = 0; r < 4; ++r) part[half][map][4 * g + r][16 * cg + c16] = s[r];
     __syncthreads();
-    const int i = tid >> 4, c = c0 + (tid & 15);                 // one channel of one sequence
-    if (i >= rows || c >= bs) return;
-    const int b = b0 + i, wc = n * bs + c;
-    const float zr = part[0][i][tid & 15] + part[2][i][tid & 15] + ld1((const uint16_t*)a.ra_b + wc);
-    const float zi = part[1][i][tid & 15] + part[3][i][tid & 15] + ld1((const uint16_t*)a.ri_b + wc);
-    float x = ld1(z + b * a.ld + W + wc), y = ld1(z + b * a.ld + wc);
-    if (a.in_b) { x += ld1((const uint16_t*)a.in_b + W + wc); y += ld1((const uint16_t*)a.in_b + wc); }
-    if (a.act) y = gelu_tanh_t<uint16_t>(y);
-    float* st = a.state + (int64_t)b * (1 + a.taps) * W + wc;
-    const float al = __builtin_amdgcn_exp2f(a.decay[wc] * LOG2E * rcp1p_exp2(-LOG2E * zr));
-    const float S = fmaf(al, st[0], __builtin_amdgcn_sqrtf(fmaxf(fmaf(-al, al, 1.0f), 0.f)) * rcp1p_exp2(-LOG2E * zi) * bf_to_f(ut[i * PR + c]));
+    if (mi >= rows || mc >= bs) return;
+    const int ci = tid % NC;
+    float al, add;
+    gate(part[0][0][mi][ci] + part[1][0][mi][ci] + br, part[0][1][mi][ci] + part[1][1][mi][ci] + bi, dec, bf_to_f(ut[mi * PR + mc]), al, add);
+    const float S = fmaf(al, S0, add);
+    if (a.act) my = gelu_tanh_t<uint16_t>(my);
     st[0] = S;
-    st[(int64_t)(1 + a.pos[b] % a.taps) * W] = x;
-    ((uint16_t*)a.o)[(int64_t)b * W + wc] = f_to_bf(S * y);
+    st[(int64_t)(1 + mpos % taps) * W] = mx;
+    ((uint16_t*)a.o)[(int64_t)mb * W + wc] = f_to_bf(S * my);
 }
 
 extern "C" int evo_rglru_step_bf16(const void* z, int64_t ld, const void* in_b, void* o, float* state, const void* conv, const void* conv_b, const void* ra,
@@ -355,12 +433,17 @@ extern "C" int evo_rglru_step_bf16(const void* z, int64_t ld, const void* in_b, 
                                    int64_t nb, int64_t taps, int64_t act, void* stream) {
     if (!rg_sizes(z, o, conv, conv_b, ra, ra_b, ri, ri_b, decay, pos, ld, B, W, nb, taps) || !state) return -1;
     const int64_t bs = W / nb;
-    if (bs % 8 || bs > 384 || ld % 8 || (((uintptr_t)z | (uintptr_t)ra | (uintptr_t)ri | (uintptr_t)in_b | (uintptr_t)conv_b | (uintptr_t)state) & 15)) return -1;
+    if (bs % 8 || bs > 384 || taps > TAPS || ld % 8 || (((uintptr_t)z | (uintptr_t)ra | (uintptr_t)ri | (uintptr_t)in_b | (uintptr_t)conv_b | (uintptr_t)state) & 15)) return -1;
     RgArgs a = {z, in_b, o, state, nullptr, conv, conv_b, ra, ra_b, ri, ri_b, decay, pos, nullptr, nullptr, nullptr,
                 ld, (int)W, (int)nb, (int)bs, (int)taps, 1, 0, 1, (int)act, (int)B};
-    const dim3 grid((unsigned)((bs + 15) / 16), (unsigned)nb, (unsigned)((B + 15) / 16));
-#define RS(KS) hipLaunchKernelGGL((rglru_step_kernel<KS>), grid, dim3(256), 0, (hipStream_t)stream, a)
+    // more channels per workgroup rebuild the convolution less often, fewer spread the weights over more workgroups
+    static const int cg_env = [] { const char* e = getenv("EVO_RG_CG"); return e ? atoi(e) : 0; }();
+    const int cg = cg_env ? cg_env : (B <= 8 ? 1 : 2);
+    const dim3 grid((unsigned)((bs + 16 * cg - 1) / (16 * cg)), (unsigned)nb, (unsigned)((B + 15) / 16));
+#define RS1(KS, CG) hipLaunchKernelGGL((rglru_step_kernel<KS, CG>), grid, dim3(256 * CG), 0, (hipStream_t)stream, a)
+#define RS(KS) do { if (cg == 1) RS1(KS, 1); else if (cg == 2) RS1(KS, 2); else RS1(KS, 4); } while (0)
     if (bs <= 64) RS(2); else if (bs <= 96) RS(3); else if (bs <= 128) RS(4); else if (bs <= 192) RS(6); else if (bs <= 256) RS(8); else RS(12);
+#undef RS1
 #undef RS
     return evo_launch_status();
 }

@@ -23,12 +23,16 @@ struct WinArgs {
 // probabilities are the next product's operand as they stand (split key order), and O^T = V^T P^T is rescaled by one factor per lane.
 // VEC: every row piece of eight elements is 16-byte aligned.
 // MAPS == 2: the two column blocks of a wave are the two maps of the same 16 queries -- rows of q and k hold [map 1 | map 2] per head --, the
-// values are shared, and the maps meet in the epilogue.  KEEP: a.keep is not zero.
-template <int KS, int DVB, int QC, bool VEC, bool KEEP, int MAPS, int MINW>
-__global__ __launch_bounds__(256, MINW) void window_attn_kernel(WinArgs a, int B) {
+// values are shared, and the maps meet in the epilogue.  KEEP: a.keep is not zero.  NW: waves
+// (8: wide heads, whose sums leave a SIMD room for two waves of one workgroup only).  NH: a tile's keys are gone through in NH parts (2: half
+// the registers for scores).
+template <int KS, int DVB, int QC, bool VEC, bool KEEP, int MAPS, int MINW, int NW = 4, int NH = 1>
+__global__ __launch_bounds__(64 * NW, MINW) void window_attn_kernel(WinArgs a, int B) {
     static_assert(MAPS == 1 || QC == 2, "two maps are two column blocks");
-    constexpr int DQ = 32 * KS, PR = MAPS * DQ + 8, PT = 64 + 4, DVP = 16 * DVB, QW = 16 * QC / MAPS, QB = 4 * QW;   // QW: queries of a wave
+    constexpr int DQ = 32 * KS, PR = MAPS * DQ + 8, PT = 64 + 4, DVP = 16 * DVB, QW = 16 * QC / MAPS, QB = NW * QW;   // QW: queries of a wave
     constexpr int KG = DQ / 64, VG = DVP / 64;                   // groups of 64 key / value dimensions
+    constexpr int KU = 8 / NW, VI = VG * 4 / NW;                 // keys per thread; groups of value dimensions per thread
+    static_assert(NW == 4 || VG % 2 == 0, "eight waves share the value groups by halves");
     __shared__ __attribute__((aligned(16))) uint16_t k_rows[64 * PR], v_cols[DVP * PT];
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int c16 = lane & 15, g = lane >> 4;
@@ -76,9 +80,10 @@ __global__ __launch_bounds__(256, MINW) void window_attn_kernel(WinArgs a, int B
         for (int db = 0; db < DVB; ++db) o[c][db] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     }
 
-    // eight threads share a row: thread (row rt, dims 8 (tid % 8) + 64 i) of keys rt and rt + 32, values of keys 2 rt and 2 rt + 1
-    const int rt = tid >> 3, ct = (tid & 7) * 8;
-    mx_u32x4 rk[MAPS * KG][2], rv[VG][2];
+    // eight threads share a row: thread (row rt, dims 8 (tid % 8) + 64 i) of keys rt and (four waves) rt + 32, values of keys 2 rt and 2 rt + 1
+    // (eight waves: rt & 31, half of the dims)
+    const int rt = tid >> 3, ct = (tid & 7) * 8, vt = rt & 31, vi0 = (rt >> 5) * VI;
+    mx_u32x4 rk[MAPS * KG][KU], rv[VI][2];
     auto any8 = [](const uint16_t* x, int nx, const uint16_t* y, int ny, int d) {       // eight dims of [x (nx) | y (ny) | zeros], any alignment
         uint32_t w[8];
 #pragma unroll
@@ -89,7 +94,7 @@ __global__ __launch_bounds__(256, MINW) void window_attn_kernel(WinArgs a, int B
     //  outputs are not stored --, so that the aligned form has no branch among its requests)
     auto load_k = [&](int j0) __attribute__((always_inline)) {
 #pragma unroll
-        for (int u = 0; u < 2; ++u) {
+        for (int u = 0; u < KU; ++u) {
             const int j = j0 + rt + 32 * u < nk ? j0 + rt + 32 * u : nk - 1;
             const uint16_t *pn = kn + j * a.ldkv, *pr_ = kr + (int64_t)j * a.dr;
 #pragma unroll
@@ -107,11 +112,11 @@ __global__ __launch_bounds__(256, MINW) void window_attn_kernel(WinArgs a, int B
     auto load_v = [&](int j0) __attribute__((always_inline)) {
 #pragma unroll
         for (int u = 0; u < 2; ++u) {
-            const int j = j0 + 2 * rt + u < nk ? j0 + 2 * rt + u : nk - 1;
+            const int j = j0 + 2 * vt + u < nk ? j0 + 2 * vt + u : nk - 1;
             const uint16_t* pv = vg + j * a.ldkv;
 #pragma unroll
-            for (int i = 0; i < VG; ++i) {
-                const int d = ct + 64 * i;
+            for (int i = 0; i < VI; ++i) {
+                const int d = ct + 64 * (vi0 + i);
                 if constexpr (!VEC) rv[i][u] = any8(pv, dv, pv, 0, d);
                 else rv[i][u] = *(const mx_u32x4*)(pv + (d < dv ? d : dv - 8));
             }
@@ -121,14 +126,15 @@ __global__ __launch_bounds__(256, MINW) void window_attn_kernel(WinArgs a, int B
 #pragma unroll
         for (int i = 0; i < MAPS * KG; ++i)
 #pragma unroll
-            for (int u = 0; u < 2; ++u) *(mx_u32x4*)(k_rows + (rt + 32 * u) * PR + ct + 64 * i) = rk[i][u];
+            for (int u = 0; u < KU; ++u) *(mx_u32x4*)(k_rows + (rt + 32 * u) * PR + ct + 64 * i) = rk[i][u];
 #pragma unroll
-        for (int i = 0; i < VG; ++i)
+        for (int i = 0; i < VI; ++i)
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
                 const uint32_t x = rv[i][0][e], y = rv[i][1][e];
-                *(uint32_t*)(v_cols + (ct + 64 * i + 2 * e) * PT + 2 * rt) = (x & 0xffffu) | y << 16;
-                *(uint32_t*)(v_cols + (ct + 64 * i + 2 * e + 1) * PT + 2 * rt) = x >> 16 | (y & 0xffff0000u);
+                uint16_t* c = v_cols + (ct + 64 * (vi0 + i) + 2 * e) * PT + 2 * vt;
+                *(uint32_t*)c = (x & 0xffffu) | y << 16;
+                *(uint32_t*)(c + PT) = x >> 16 | (y & 0xffff0000u);
             }
     };
 
@@ -148,15 +154,18 @@ __global__ __launch_bounds__(256, MINW) void window_attn_kernel(WinArgs a, int B
         next = after(j0);
         const bool more = next <= j_hi;
         const bool mine = j0 <= w_last && (j0 + 63 > w_first - a.window || (KEEP && j0 < a.keep));   // some query of this wave sees some key of the tile
-        f32x4_t s[QC][4];
+        constexpr int NJ = 4 / NH;                               // 16-key blocks of a part
+#pragma unroll
+        for (int hh = 0; hh < NH; ++hh) {
+        f32x4_t s[QC][NJ];
         if (mine) {
 #pragma unroll
-            for (int jb = 0; jb < 4; ++jb) {
+            for (int jb = 0; jb < NJ; ++jb) {
 #pragma unroll
                 for (int c = 0; c < QC; ++c) s[c][jb] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
                 for (int ks = 0; ks < KS; ++ks) {
-                    const uint16_t* kp = k_rows + (16 * jb + c16) * PR + 32 * ks + 8 * g;
+                    const uint16_t* kp = k_rows + (16 * (hh * NJ + jb) + c16) * PR + 32 * ks + 8 * g;
                     const mx_frag kf = __builtin_bit_cast(mx_frag, *(const uint4*)kp);
 #pragma unroll
                     for (int c = 0; c < QC; ++c)
@@ -167,25 +176,25 @@ __global__ __launch_bounds__(256, MINW) void window_attn_kernel(WinArgs a, int B
         }
         // the next tile's requests go out in two parts, between the phases: with all of them ahead of the scores the register file spills
         __builtin_amdgcn_sched_barrier(0);
-        if (more) load_k(next);
+        if (hh == NH - 1 && more) load_k(next);
         __builtin_amdgcn_sched_barrier(0);
-        mx_frag pf[QC][2];
+        mx_frag pf[QC][NJ / 2];
         if (mine) {
             if (j0 + 63 > w_first || (j0 <= w_last - a.window && (!KEEP || j0 + 63 >= a.keep))) {   // the tile holds an edge of some query's window
 #pragma unroll
                 for (int c = 0; c < QC; ++c)
 #pragma unroll
-                    for (int jb = 0; jb < 4; ++jb)
+                    for (int jb = 0; jb < NJ; ++jb)
 #pragma unroll
                         for (int r = 0; r < 4; ++r) {
-                            const int j = j0 + 16 * jb + 4 * g + r, age = qi[c] - j;
+                            const int j = j0 + 16 * (hh * NJ + jb) + 4 * g + r, age = qi[c] - j;
                             s[c][jb][r] = age >= 0 && (age < a.window || (KEEP && j < a.keep)) ? s[c][jb][r] * sc2 : -INFINITY;
                         }
             } else {
 #pragma unroll
                 for (int c = 0; c < QC; ++c)
 #pragma unroll
-                    for (int jb = 0; jb < 4; ++jb)
+                    for (int jb = 0; jb < NJ; ++jb)
 #pragma unroll
                         for (int r = 0; r < 4; ++r) s[c][jb][r] *= sc2;
             }
@@ -193,7 +202,7 @@ __global__ __launch_bounds__(256, MINW) void window_attn_kernel(WinArgs a, int B
             for (int c = 0; c < QC; ++c) {
                 float top = mx[c];
 #pragma unroll
-                for (int jb = 0; jb < 4; ++jb) top = fmaxf(top, fmaxf(fmaxf(s[c][jb][0], s[c][jb][1]), fmaxf(s[c][jb][2], s[c][jb][3])));
+                for (int jb = 0; jb < NJ; ++jb) top = fmaxf(top, fmaxf(fmaxf(s[c][jb][0], s[c][jb][1]), fmaxf(s[c][jb][2], s[c][jb][3])));
                 top = fmaxf(top, __shfl_xor(top, 16, 64));
                 top = fmaxf(top, __shfl_xor(top, 32, 64));
                 if (__builtin_amdgcn_ballot_w64(top > mx[c])) {          // the running maximum moved in some column: rescale
@@ -205,9 +214,9 @@ __global__ __launch_bounds__(256, MINW) void window_attn_kernel(WinArgs a, int B
 #pragma unroll
                         for (int r = 0; r < 4; ++r) o[c][db][r] *= f;
                 }
-                uint32_t w[8];
+                uint32_t w[2 * NJ];
 #pragma unroll
-                for (int jb = 0; jb < 4; ++jb) {
+                for (int jb = 0; jb < NJ; ++jb) {
                     float e[4];
 #pragma unroll
                     for (int r = 0; r < 4; ++r) {
@@ -217,23 +226,24 @@ __global__ __launch_bounds__(256, MINW) void window_attn_kernel(WinArgs a, int B
                     w[2 * jb] = pack_bf2(e[0], e[1]);
                     w[2 * jb + 1] = pack_bf2(e[2], e[3]);
                 }
-                pf[c][0] = frag_of(w[0], w[1], w[2], w[3]);
-                pf[c][1] = frag_of(w[4], w[5], w[6], w[7]);
+#pragma unroll
+                for (int jj = 0; jj < NJ / 2; ++jj) pf[c][jj] = frag_of(w[4 * jj], w[4 * jj + 1], w[4 * jj + 2], w[4 * jj + 3]);
             }
         }
         __builtin_amdgcn_sched_barrier(0);
-        if (more) load_v(next);
+        if (hh == NH - 1 && more) load_v(next);
         __builtin_amdgcn_sched_barrier(0);
         if (mine) {
 #pragma unroll
-            for (int jj = 0; jj < 2; ++jj)
+            for (int jj = 0; jj < NJ / 2; ++jj)
 #pragma unroll
                 for (int db = 0; db < DVB; ++db) {
-                    const mx_frag vf = frag_split(v_cols + (16 * db + c16) * PT + 32 * jj + 4 * g);
+                    const mx_frag vf = frag_split(v_cols + (16 * db + c16) * PT + 32 * (hh * (NJ / 2) + jj) + 4 * g);
 #pragma unroll
                     for (int c = 0; c < QC; ++c) o[c][db] = mfma16(vf, pf[c][jj], o[c][db]);
                     if ((db & 3) == 3) __builtin_amdgcn_sched_barrier(0);
                 }
+        }
         }
         __syncthreads();
     }
@@ -359,16 +369,17 @@ extern "C" int evo_window_attn(const void* q, int64_t ldq, const void* kn, const
     if (!f32 && mfma && dq <= (maps == 2 ? 128 : 256) && dv <= 256) {
         const bool vec = dn % 8 == 0 && dr % 8 == 0 && dv % 8 == 0 && ldq % 8 == 0 && ldkv % 8 == 0 &&
                          (((uintptr_t)q | (uintptr_t)kn | (uintptr_t)v | (uintptr_t)kr) & 15) == 0;
-#define WA1(KS, DVB, QC, VEC, KEEP, MAPS, MINW)                                                                            \
+#define WA1(KS, DVB, QC, VEC, KEEP, MAPS, MINW, NW)                                                                        \
     do {                                                                                                                   \
-        a.n_qb = (int)((max_q + 64 * QC / MAPS - 1) / (64 * QC / MAPS));                                                   \
+        a.n_qb = (int)((max_q + 16 * NW * QC / MAPS - 1) / (16 * NW * QC / MAPS));                                         \
         const int64_t items = (int64_t)a.n_qb * H * B;                                                                     \
         if (items > 0x7ffffff0) return -1;                                                                                 \
-        hipLaunchKernelGGL((window_attn_kernel<KS, DVB, QC, VEC, KEEP, MAPS, MINW>), dim3((unsigned)((items + 7) / 8 * 8)), dim3(256), 0, s, a, (int)B); \
+        hipLaunchKernelGGL((window_attn_kernel<KS, DVB, QC, VEC, KEEP, MAPS, MINW, NW, (MAPS == 2 && NW == 8 ? 2 : 1)>), dim3((unsigned)((items + 7) / 8 * 8)), dim3(64 * NW), 0, s, a, (int)B); \
     } while (0)
-#define WA(KS, DVB, QC, VEC, MAPS, MINW) do { if (kp) WA1(KS, DVB, QC, VEC, true, MAPS, MINW); else WA1(KS, DVB, QC, VEC, false, MAPS, MINW); } while (0)
+#define WAN(KS, DVB, QC, VEC, MAPS, MINW, NW) do { if (kp) WA1(KS, DVB, QC, VEC, true, MAPS, MINW, NW); else WA1(KS, DVB, QC, VEC, false, MAPS, MINW, NW); } while (0)
+#define WA(KS, DVB, QC, VEC, MAPS, MINW) WAN(KS, DVB, QC, VEC, MAPS, MINW, 4)
 #define WAV(KS, QC) do { if (dv <= 64) WA(KS, 4, QC, true, 1, 2); else if (dv <= 128) WA(KS, 8, QC, true, 1, 2); else WA(KS, 16, 1, true, 1, 2); } while (0)
-#define WA2(KS) do { if (dv <= 64) WA(KS, 4, 2, true, 2, 2); else if (dv <= 128) WA(KS, 8, 2, true, 2, 2); else WA(KS, 16, 2, true, 2, 1); } while (0)
+#define WA2(KS) do { if (dv <= 64) WA(KS, 4, 2, true, 2, 2); else if (dv <= 128) WA(KS, 8, 2, true, 2, 2); else WAN(KS, 16, 2, true, 2, 2, 8); } while (0)
         if (maps == 2) { if (!vec) WA(4, 16, 2, false, 2, 1); else if (dq <= 64) WA2(2); else WA2(4); }
         else if (!vec) { if (dq <= 64 && dv <= 64) WA(2, 4, 2, false, 1, 2); else WA(8, 16, 1, false, 1, 2); }
         else if (dq <= 64) WAV(2, 2);
@@ -376,8 +387,8 @@ extern "C" int evo_window_attn(const void* q, int64_t ldq, const void* kn, const
         else if (dq <= 192) {                                    // (kept tokens cost registers: one column block)
             if (dv <= 64) WA(6, 4, 2, true, 1, 2);
             else if (dv > 128) WA(6, 16, 1, true, 1, 2);
-            else if (kp) WA1(6, 8, 1, true, true, 1, 2);
-            else WA1(6, 8, 2, true, false, 1, 2);
+            else if (kp) WA1(6, 8, 1, true, true, 1, 2, 4);
+            else WA1(6, 8, 2, true, false, 1, 2, 4);
         }
         else if (dv <= 64) WA(8, 4, 1, true, 1, 2);
         else if (dv <= 128) WA(8, 8, 1, true, 1, 2);
@@ -385,6 +396,7 @@ extern "C" int evo_window_attn(const void* q, int64_t ldq, const void* kn, const
 #undef WA2
 #undef WAV
 #undef WA
+#undef WAN
 #undef WA1
         return evo_launch_status();
     }

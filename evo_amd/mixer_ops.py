@@ -439,10 +439,10 @@ class MixerOps:
         return dtype == torch.bfloat16 and bs % 8 == 0 and bs <= 384 and taps <= 4
 
     @staticmethod
-    def rglru_segment(L: int, walkers: int, target: int = 192) -> int:
-        """Tokens per segment: one segment while the walking workgroups fill most of the chip, else enough segments for that (a segment's state
-        costs another pass over its gates)."""
-        want = max(1, (target + walkers - 1) // walkers)
+    def rglru_segment(L: int, walkers: int, target: int = 256) -> int:
+        """Tokens per segment: one segment while the walking workgroups fill most of the chip, else as many as give every CU one (a segment's
+        state costs another pass over its gates)."""
+        want = max(1, target // walkers) if walkers <= target * 5 // 8 else 1
         return max(256, (L + want * 64 - 1) // (want * 64) * 64) if want > 1 else (L + 63) // 64 * 64
 
     def rglru(self, z: torch.Tensor, in_b: Optional[torch.Tensor], act: bool, W: int, conv: torch.Tensor, conv_b: torch.Tensor, ra, ra_b, ri, ri_b,
