@@ -34,10 +34,16 @@ __device__ __forceinline__ uint4 ld_stream(const uint4* p) {
 // SPLIT: the four waves of a workgroup share the SAME R rows and each takes every fourth 64-vector slice of K (the
 // partial sums meet in LDS).  Used for the narrow layers (N <= 4096: out_filter_dense, out_proj, l3), where one wave
 // per R rows leaves the chip with too few loads in flight: 3.3 -> see tools/bench_gemv.py.
+// an ungated feed-forward's activation on the way out: act 3 = square of relu, else none
+__device__ __forceinline__ float out_act(float o, int act) {
+    const float z = fmaxf(o, 0.f);
+    return act == 3 ? z * z : o;
+}
+
 template <int M, int R, bool SPLIT>
 __global__ __launch_bounds__(256) void gemv_kernel(const uint4* __restrict__ x, const uint4* __restrict__ w,
                                                    const uint16_t* __restrict__ bias, const uint16_t* res,
-                                                   uint16_t* y, int N, int nvec) {   // res may alias y
+                                                   uint16_t* y, int N, int nvec, int act) {   // res may alias y
     __shared__ float part[SPLIT ? 4 * R * M : 1];
     const int lane = threadIdx.x & 63;
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
@@ -121,7 +127,7 @@ __global__ __launch_bounds__(256) void gemv_kernel(const uint4* __restrict__ x, 
                 for (int m = 0; m < M; ++m) {
                     float o = acc[r][m] + b;
                     if (res) o += bf_to_f(pf_r[r][m]);
-                    y[(int64_t)m * N + n] = f_to_bf(o);
+                    y[(int64_t)m * N + n] = f_to_bf(out_act(o, act));
                 }
             }
         }
@@ -806,7 +812,7 @@ typedef float gv_f32x4 __attribute__((ext_vector_type(4)));
 template <int MT, int NT>
 __global__ __launch_bounds__(512) void skinny_mfma_kernel(const uint4* __restrict__ x, const uint4* __restrict__ w,
                                                           const uint16_t* __restrict__ bias, const uint16_t* res,
-                                                          uint16_t* y, int M, int N, int nvec) {   // res may alias y
+                                                          uint16_t* y, int M, int N, int nvec, int act) {   // res may alias y
     static_assert(MT * NT <= 8, "one reducing wave per (n tile, m tile)");
     __shared__ gv_f32x4 part[NT * MT][8][64];
     const int lane = threadIdx.x & 63;
@@ -884,7 +890,7 @@ __global__ __launch_bounds__(512) void skinny_mfma_kernel(const uint4* __restric
                 if (n < N) {
                     float o = a_[r] + (bias ? bf_to_f(bias[n]) : 0.f);
                     if (res) o += bf_to_f(res[(int64_t)m * N + n]);
-                    y[(int64_t)m * N + n] = f_to_bf(o);
+                    y[(int64_t)m * N + n] = f_to_bf(out_act(o, act));
                 }
             }
         }
@@ -900,7 +906,7 @@ __global__ __launch_bounds__(512) void skinny_mfma_kernel(const uint4* __restric
 template <int MT, int WAVES>
 __global__ __launch_bounds__(64 * WAVES) void skinny_n_kernel(const uint4* __restrict__ x, const uint4* __restrict__ w,
                                                               const uint16_t* __restrict__ bias, const uint16_t* res,
-                                                              uint16_t* y, int M, int N, int nvec) {   // res may alias y
+                                                              uint16_t* y, int M, int N, int nvec, int act) {   // res may alias y
     constexpr int KC = 8, ROWB = KC * 64 + 16;                   // steps per chunk; LDS bytes per x row (512 + 16 pad)
     constexpr int XL = (MT * 16 * KC * 4 + 64 * WAVES - 1) / (64 * WAVES);   // 16-byte pieces of an x chunk per thread
     __shared__ __attribute__((aligned(16))) unsigned char xs[2][MT * 16 * ROWB];
@@ -979,7 +985,7 @@ __global__ __launch_bounds__(64 * WAVES) void skinny_n_kernel(const uint4* __res
                 if (n < N) {
                     float o = acc[t][r] + (bias ? bf_to_f(bias[n]) : 0.f);
                     if (res) o += bf_to_f(res[(int64_t)m * N + n]);
-                    y[(int64_t)m * N + n] = f_to_bf(o);
+                    y[(int64_t)m * N + n] = f_to_bf(out_act(o, act));
                 }
             }
         }
@@ -1128,7 +1134,7 @@ __global__ __launch_bounds__(64 * WAVES) void skinny_nw_kernel(const uint4* __re
                 if (n < N) {
                     float o = acc[t][r] + (bias ? bf_to_f(bias[n]) : 0.f);
                     if (res) o += bf_to_f(res[(int64_t)m * N + n]);
-                    y[(int64_t)m * N + n] = f_to_bf(o);
+                    y[(int64_t)m * N + n] = f_to_bf(out_act(o, act));
                 }
             }
         }
@@ -1137,7 +1143,7 @@ __global__ __launch_bounds__(64 * WAVES) void skinny_nw_kernel(const uint4* __re
 
 // y [M, N] = sum over slices of ws [slices][M][N] (in slice order: deterministic) + bias + residual, one rounding; a thread owns four columns
 __global__ __launch_bounds__(256) void skinny_reduce_kernel(const float* __restrict__ ws, const uint16_t* __restrict__ bias, const uint16_t* res,
-                                                            uint16_t* y, int M, int N, int slices) {   // res may alias y
+                                                            uint16_t* y, int M, int N, int slices, int act) {   // res may alias y
     const int64_t q = (int64_t)blockIdx.x * 256 + threadIdx.x, total = (int64_t)M * N / 4;
     if (q >= total) return;
     const int64_t e = q * 4;
@@ -1148,14 +1154,14 @@ __global__ __launch_bounds__(256) void skinny_reduce_kernel(const float* __restr
     if (bias) { const uint2 b = *(const uint2*)(bias + n); o[0] += bf_lo(b.x); o[1] += bf_hi(b.x); o[2] += bf_lo(b.y); o[3] += bf_hi(b.y); }
     if (res) { const uint2 r = *(const uint2*)(res + e); o[0] += bf_lo(r.x); o[1] += bf_hi(r.x); o[2] += bf_lo(r.y); o[3] += bf_hi(r.y); }
     uint2 out;
-    out.x = pack_bf2(o[0], o[1]);
-    out.y = pack_bf2(o[2], o[3]);
+    out.x = pack_bf2(out_act(o[0], act), out_act(o[1], act));
+    out.y = pack_bf2(out_act(o[2], act), out_act(o[3], act));
     *(uint2*)(y + e) = out;
 }
 
 template <int M>
 static void gemv_launch(const void* x, const void* w, const void* bias, const void* res, void* y, int64_t N, int64_t K,
-                        hipStream_t s) {
+                        int act, hipStream_t s) {
     // rows per wave.  Measured (tools/bench_gemv.py, MI355X): R=4 wins for every M (R=8 starves the chip of
     // waves at N=4096; R=2 doubles the L2 re-reads of x): 4.9-5.4 TB/s at M=1-2, 3.0-3.6 TB/s at M=8.
 #ifndef GEMV_R_A
@@ -1171,10 +1177,10 @@ static void gemv_launch(const void* x, const void* w, const void* bias, const vo
     const int64_t waves = (N + R - 1) / R;
     if (N <= 4096 && K >= 2048)
         hipLaunchKernelGGL((gemv_kernel<M, R, true>), dim3((unsigned)waves), dim3(256), 0, s, (const uint4*)x,
-                           (const uint4*)w, (const uint16_t*)bias, (const uint16_t*)res, (uint16_t*)y, (int)N, (int)(K / 8));
+                           (const uint4*)w, (const uint16_t*)bias, (const uint16_t*)res, (uint16_t*)y, (int)N, (int)(K / 8), act);
     else
         hipLaunchKernelGGL((gemv_kernel<M, R, false>), dim3((unsigned)((waves + 3) / 4)), dim3(256), 0, s, (const uint4*)x,
-                           (const uint4*)w, (const uint16_t*)bias, (const uint16_t*)res, (uint16_t*)y, (int)N, (int)(K / 8));
+                           (const uint4*)w, (const uint16_t*)bias, (const uint16_t*)res, (uint16_t*)y, (int)N, (int)(K / 8), act);
 }
 
 extern "C" int evo_norm_linear_small_m_bf16(const void* x, const void* scale, const void* w, const void* bias, void* y,
@@ -1312,9 +1318,9 @@ extern "C" int evo_norm_mlp_gate_small_m_bf16(const void* x, const void* scale, 
 }
 
 extern "C" int evo_linear_small_m_bf16(const void* x, const void* w, const void* bias, const void* residual, void* y,
-                                       int64_t M, int64_t N, int64_t K, void* ws, int64_t ws_bytes, void* stream) {
+                                       int64_t M, int64_t N, int64_t K, void* ws, int64_t ws_bytes, int64_t act, void* stream) {
     if (M < 1 || M > 64 || N <= 0 || K <= 0 || K % 8 != 0 || N > 0x7fffffff - 16) return -1;
-    if (M > 8 && K % 32 != 0) return -1;
+    if ((M > 8 && K % 32 != 0) || (act != 0 && act != 3)) return -1;
     hipStream_t s = (hipStream_t)stream;
     if (M >= 5 && K % 32 == 0) {
         // two n tiles per workgroup (every x fragment feeds two weight fragments) where that still leaves a workgroup or more per CU
@@ -1345,14 +1351,14 @@ extern "C" int evo_linear_small_m_bf16(const void* x, const void* w, const void*
                 if (M <= 16) EVO_SNK(1); else if (M <= 32) EVO_SNK(2); else if (M <= 48) EVO_SNK(3); else EVO_SNK(4);
 #undef EVO_SNK
                 hipLaunchKernelGGL(skinny_reduce_kernel, dim3((unsigned)((M * N / 4 + 255) / 256)), dim3(256), 0, s, (const float*)ws, (const uint16_t*)bias,
-                                   (const uint16_t*)residual, (uint16_t*)y, (int)M, (int)N, (int)slices);
+                                   (const uint16_t*)residual, (uint16_t*)y, (int)M, (int)N, (int)slices, (int)act);
                 return evo_launch_status();
             }
         }
         if (K % 256 == 0 && N >= 8192 && nw_env && M >= nwm_env && ns_env < 0) {
             const int wv = nww_env ? nww_env : (N >= 256 * 64 ? 4 : (N >= 256 * 48 ? 3 : (N >= 256 * 32 ? 2 : 4)));   // a workgroup or more per CU where N allows
 #define EVO_SNW(MT, WV) hipLaunchKernelGGL((skinny_nw_kernel<MT, WV>), dim3((unsigned)((N + 16 * WV - 1) / (16 * WV))), dim3(64 * WV), 0, s, (const uint4*)x, \
-                                           (const uint4*)w, (const uint16_t*)bias, (const uint16_t*)residual, (uint16_t*)y, (int)M, (int)N, (int)(K / 8))
+                                           (const uint4*)w, (const uint16_t*)bias, (const uint16_t*)residual, (uint16_t*)y, (int)M, (int)N, (int)(K / 8), (float*)nullptr, 0, (int)act)
             if (wv == 4) { if (M <= 16) EVO_SNW(1, 4); else if (M <= 32) EVO_SNW(2, 4); else if (M <= 48) EVO_SNW(3, 4); else EVO_SNW(4, 4); }
             else if (wv == 3) { if (M <= 16) EVO_SNW(1, 3); else if (M <= 32) EVO_SNW(2, 3); else if (M <= 48) EVO_SNW(3, 3); else EVO_SNW(4, 3); }
             else { if (M <= 16) EVO_SNW(1, 2); else if (M <= 32) EVO_SNW(2, 2); else if (M <= 48) EVO_SNW(3, 2); else EVO_SNW(4, 2); }
@@ -1362,7 +1368,7 @@ extern "C" int evo_linear_small_m_bf16(const void* x, const void* w, const void*
         if (waves_n && K % 256 == 0) {
 #define EVO_SN(MT, WV)                                                                                                     \
             hipLaunchKernelGGL((skinny_n_kernel<MT, WV>), dim3((unsigned)((N + 16 * WV - 1) / (16 * WV))), dim3(64 * WV), 0, s, (const uint4*)x,  \
-                               (const uint4*)w, (const uint16_t*)bias, (const uint16_t*)residual, (uint16_t*)y, (int)M, (int)N, (int)(K / 8))
+                               (const uint4*)w, (const uint16_t*)bias, (const uint16_t*)residual, (uint16_t*)y, (int)M, (int)N, (int)(K / 8), (int)act)
             if (waves_n == 4) { if (M <= 16) EVO_SN(1, 4); else if (M <= 32) EVO_SN(2, 4); else if (M <= 48) EVO_SN(3, 4); else EVO_SN(4, 4); }
             else { if (M <= 16) EVO_SN(1, 2); else if (M <= 32) EVO_SN(2, 2); else if (M <= 48) EVO_SN(3, 2); else EVO_SN(4, 2); }
 #undef EVO_SN
@@ -1370,21 +1376,21 @@ extern "C" int evo_linear_small_m_bf16(const void* x, const void* w, const void*
         }
 #define EVO_SK(MT, NT)                                                                                                     \
         hipLaunchKernelGGL((skinny_mfma_kernel<MT, NT>), dim3((unsigned)((N + 16 * NT - 1) / (16 * NT))), block, 0, s, (const uint4*)x, (const uint4*)w, \
-                           (const uint16_t*)bias, (const uint16_t*)residual, (uint16_t*)y, (int)M, (int)N, (int)(K / 8))
+                           (const uint16_t*)bias, (const uint16_t*)residual, (uint16_t*)y, (int)M, (int)N, (int)(K / 8), (int)act)
         if (nt == 2) { if (M <= 16) EVO_SK(1, 2); else if (M <= 32) EVO_SK(2, 2); else if (M <= 48) EVO_SK(3, 2); else EVO_SK(4, 2); }
         else { if (M <= 16) EVO_SK(1, 1); else if (M <= 32) EVO_SK(2, 1); else if (M <= 48) EVO_SK(3, 1); else EVO_SK(4, 1); }
 #undef EVO_SK
         return evo_launch_status();
     }
     switch (M) {
-        case 1: gemv_launch<1>(x, w, bias, residual, y, N, K, s); break;
-        case 2: gemv_launch<2>(x, w, bias, residual, y, N, K, s); break;
-        case 3: gemv_launch<3>(x, w, bias, residual, y, N, K, s); break;
-        case 4: gemv_launch<4>(x, w, bias, residual, y, N, K, s); break;
-        case 5: gemv_launch<5>(x, w, bias, residual, y, N, K, s); break;
-        case 6: gemv_launch<6>(x, w, bias, residual, y, N, K, s); break;
-        case 7: gemv_launch<7>(x, w, bias, residual, y, N, K, s); break;
-        default: gemv_launch<8>(x, w, bias, residual, y, N, K, s); break;
+        case 1: gemv_launch<1>(x, w, bias, residual, y, N, K, (int)act, s); break;
+        case 2: gemv_launch<2>(x, w, bias, residual, y, N, K, (int)act, s); break;
+        case 3: gemv_launch<3>(x, w, bias, residual, y, N, K, (int)act, s); break;
+        case 4: gemv_launch<4>(x, w, bias, residual, y, N, K, (int)act, s); break;
+        case 5: gemv_launch<5>(x, w, bias, residual, y, N, K, (int)act, s); break;
+        case 6: gemv_launch<6>(x, w, bias, residual, y, N, K, (int)act, s); break;
+        case 7: gemv_launch<7>(x, w, bias, residual, y, N, K, (int)act, s); break;
+        default: gemv_launch<8>(x, w, bias, residual, y, N, K, (int)act, s); break;
     }
     return evo_launch_status();
 }

@@ -235,9 +235,12 @@ class MixerOps:
         return a
 
     def linear_act(self, x: torch.Tensor, w: torch.Tensor, act: str, act_cols: int, b: Optional[torch.Tensor] = None) -> torch.Tensor:
-        """x @ w^T (+ b) with an activation on the first `act_cols` columns; prefill-sized batches in the dense layer's epilogue."""
+        """x @ w^T (+ b) with an activation on the first `act_cols` columns; in the dense layer's epilogue for prefill-sized
+        batches and, the square of relu on all columns, for decode-sized ones."""
         M, K = x.shape
         N = w.shape[0]
+        if act == "relu2" and act_cols == N and self._use_small_m(x, w):
+            return self._linear_small_m(x, w, b, None, act=ACTIVATIONS[act])
         if (self._take_mfma(False) and self.mfma_linear_ok(x, w) and not self._use_small_m(x, w) and act_cols % 256 == 0 and K >= 128
                 and M * K * 2 < 0xffffffff and N * K * 2 < 0xffffffff):
             r = self._tail_rows(x, w)
@@ -410,8 +413,8 @@ class MixerOps:
 
     @staticmethod
     def heads_split(groups: int, ring: int, cus: int = 256) -> int:
-        """Parts of the cache in the decode kernel: two workgroups per CU, at least 128 slots (one round of a workgroup's waves) each."""
-        return max(1, min((ring + 127) // 128, (2 * cus + groups - 1) // groups, 64))
+        """Parts of the cache in the decode kernel: a workgroup per CU, at least 128 slots (one round of a workgroup's waves) each."""
+        return max(1, min((ring + 127) // 128, (cus + groups - 1) // groups, 64))
 
     def heads_decode(self, z: torch.Tensor, cache: torch.Tensor, pos: torch.Tensor, heads: int, kv_heads: int, maps: int, dim: int, dv: int, scale: float,
                      lam: float, gain: float, eps: float, n_split: Optional[int] = None) -> torch.Tensor:

@@ -52,7 +52,7 @@ extern "C" {
  *  11: evo_mlp_gate_mfma_bf16 and evo_mlp_gate_small_m_bf16 gained `act` (gate function: 0 exact-erf GELU, 1 SiLU); evo_linear_silu_mfma_bf16, the evo_postnorm_* launches and the mixers library added:
  *      fp32-residual-stream kernels, decayed linear attention, latent attention (the last section of this file).
  *  12: evo_linear_act_mfma_bf16 (bias, three activations) and evo_act_cols take the places of evo_linear_silu_mfma_bf16 and evo_silu_cols; the
- *      evo_postnorm_* launches gained the norm of the sum (`alpha`, `sum`) and the plain one an activation; evo_window_attn gained grouped key heads,
+ *      evo_postnorm_* launches gained the norm of the sum (`alpha`, `sum`) and the plain one an activation, as did evo_linear_small_m_bf16; evo_window_attn gained grouped key heads,
  *      kept first tokens and two maps; evo_sum_norm, evo_heads_* and evo_rglru_* added. */
 #define EVO_ABI_VERSION 12
 int evo_abi_version(void);
@@ -247,9 +247,10 @@ int evo_attn_decode_bf16(const void* q, const void* k, const void* v, void* o,
  * (17-64 rows: the pooled decode step of 17-64 live streams); `residual` may alias `y`.  From 5 rows on layers with N >= 8192 and K % 256 == 0 the
  * weight is requested in whole 512-byte row pieces and the x rows of a 256-k chunk are shared by the workgroup's waves through LDS (csrc/gemv.hip
  * skinny_nw_kernel).  `ws` (ABI 10; may be NULL): a 16-byte aligned fp32 workspace of `ws_bytes` >= 8 M N 4 bytes lets the narrow layers (N < 8192) at
- * 17-64 rows split K over workgroups -- partial sums through ws, added in a fixed order by a second small launch; without it they run the k-split form. */
+ * 17-64 rows split K over workgroups -- partial sums through ws, added in a fixed order by a second small launch; without it they run the k-split form.
+ * act 3: the square of relu before the rounding (0: none). */
 int evo_linear_small_m_bf16(const void* x, const void* w, const void* bias, const void* residual, void* y,
-                            int64_t M, int64_t N, int64_t K, void* ws, int64_t ws_bytes, void* stream);
+                            int64_t M, int64_t N, int64_t K, void* ws, int64_t ws_bytes, int64_t act, void* stream);
 
 /* ---- dense layer on the MFMA pipe (prefill) --------------------------------------------------------------
  * replaces the cuBLAS nn.Linear GEMMs of the attention block: Wqkv (with bias) and out_proj (+ residual)

@@ -202,7 +202,8 @@ def test_norm_of_the_sum_in_the_next_layers_launch(ops, M, K, N):
 @TYPES
 @pytest.mark.parametrize("act,fn", [("silu", V.silu), ("gelu_tanh", R.gelu_tanh), ("relu2", R.squared_relu)])
 @pytest.mark.parametrize("bias", [False, True])
-@pytest.mark.parametrize("M,N,K,n", [(3, 70, 52, 33), (20, 512, 128, 256), (300, 512, 192, 256), (300, 512, 192, 512), (300, 512, 192, 200), (5129, 512, 128, 256), (40, 1280, 256, 1280)])
+@pytest.mark.parametrize("M,N,K,n", [(3, 70, 52, 33), (20, 512, 128, 256), (300, 512, 192, 256), (300, 512, 192, 512), (300, 512, 192, 200), (5129, 512, 128, 256), (40, 1280, 256, 1280),
+                                     (1, 70, 64, 70), (4, 4096, 2048, 4096), (7, 128, 72, 128), (9, 8192, 256, 8192), (33, 8192, 256, 8192), (33, 2048, 8192, 2048), (64, 320, 96, 320)])
 def test_linear_with_activation(ops, dt, act, fn, bias, M, N, K, n):
     x, w, b = rnd(M, K, seed=1, dt=dt), rnd(N, K, seed=2, dt=dt, scale=2.0 / math.sqrt(K)), rnd(N, seed=3, dt=dt)
     got = ops.linear_act(x.to(DEV), w.to(DEV), act, n, b.to(DEV) if bias else None)
