@@ -10,7 +10,6 @@
 // (1) every segment's decay product and end state from zero, (2) a scan over segments, (3) outputs.
 #include "mixers_common.h"
 #include "../../include/evo_mi355x.h"
-#include <cstdlib>
 #include <type_traits>
 
 #define LOG2E 1.4426950408889634f
@@ -359,17 +358,23 @@ __global__ __launch_bounds__(256 * CG) void rglru_step_kernel(RgArgs a) {
     const float S0 = st[0], dec = a.decay[wc] * LOG2E, br = ld1((const uint16_t*)a.ra_b + wc), bi = ld1((const uint16_t*)a.ri_b + wc);
     float mx = ld1(z + mb * a.ld + W + wc), my = ld1(z + mb * a.ld + wc);
     if (a.in_b) { mx += ld1((const uint16_t*)a.in_b + W + wc); my += ld1((const uint16_t*)a.in_b + wc); }
-    const int64_t mpos = a.pos[mb];
+    const uint32_t mpos = (uint32_t)a.pos[mb];
 
-    for (int i = tid; i < (taps + 1) * KP; i += NT) {
-        const int t = i / KP, c = i - t * KP;
-        cw[i] = t < taps && c < bs ? ld1((const uint16_t*)a.conv + (int64_t)(n * bs + c) * taps + t) : 0.f;
+    constexpr int CI = ((TAPS + 1) * KP + NT - 1) / NT;          // (all requests first: one memory latency)
+    float tap[CI];
+#pragma unroll
+    for (int k = 0; k < CI; ++k) {
+        const int i = tid + NT * k, t = i / KP, c = i % KP;
+        tap[k] = ld1((const uint16_t*)a.conv + (int64_t)(n * bs + (c < bs ? c : bs - 1)) * taps + (t < taps ? t : 0));
+        if (t >= taps || c >= bs) tap[k] = 0.f;
     }
     constexpr int ND = KP / 8, IT = (16 * ND + NT - 1) / NT;     // runs of eight channels of one sequence, per thread
     float acc[IT][8], h[IT][TAPS][8], x[IT][8];
+    uint32_t p[IT];                                              // (positions are far below 2^31)
 #pragma unroll
     for (int k = 0; k < IT; ++k) {
         const int it = tid + NT * k, i = it / ND, d = 8 * (it % ND), b = b0 + (i < rows ? i : rows - 1), dc = d < bs ? d : 0;
+        p[k] = (uint32_t)a.pos[b];
         vec_io<uint16_t, 8>::load(z + b * a.ld + W + n * bs + dc, x[k]);
         vec_io<uint16_t, 8>::load((const uint16_t*)a.conv_b + n * bs + dc, acc[k]);
 #pragma unroll
@@ -382,13 +387,15 @@ __global__ __launch_bounds__(256 * CG) void rglru_step_kernel(RgArgs a) {
             for (int e = 0; e < 8; ++e) x[k][e] += ib[e];
         }
     }
+#pragma unroll
+    for (int k = 0; k < CI; ++k)
+        if (tid + NT * k < (TAPS + 1) * KP) cw[tid + NT * k] = tap[k];
     __syncthreads();
 #pragma unroll
     for (int k = 0; k < IT; ++k) {
         const int it = tid + NT * k, i = it / ND, d = 8 * (it % ND);
         if (it >= 16 * ND) break;
-        const int64_t p = a.pos[b0 + (i < rows ? i : rows - 1)];
-        const int cur = (int)(p % taps);
+        const int cur = (int)(p[k] % (uint32_t)taps);
         auto add = [&](int row, const float* v) {
             float w[8];
             vec_io<float, 8>::load(cw + row * KP + d, w);
@@ -399,7 +406,7 @@ __global__ __launch_bounds__(256 * CG) void rglru_step_kernel(RgArgs a) {
 #pragma unroll
         for (int t = 0; t < TAPS; ++t) {
             const int back = cur - t + (cur < t ? taps : 0);     // tokens between this one and the row's
-            const bool have = t < taps && back > 0 && p - back >= 0;
+            const bool have = t < taps && back > 0 && (uint32_t)back <= p[k];
             float v[8];
 #pragma unroll
             for (int e = 0; e < 8; ++e) v[e] = have ? h[k][t][e] : 0.f;
@@ -424,7 +431,7 @@ __global__ __launch_bounds__(256 * CG) void rglru_step_kernel(RgArgs a) {
     const float S = fmaf(al, S0, add);
     if (a.act) my = gelu_tanh_t<uint16_t>(my);
     st[0] = S;
-    st[(int64_t)(1 + mpos % taps) * W] = mx;
+    st[(int64_t)(1 + mpos % (uint32_t)taps) * W] = mx;
     ((uint16_t*)a.o)[(int64_t)mb * W + wc] = f_to_bf(S * my);
 }
 
@@ -437,12 +444,12 @@ extern "C" int evo_rglru_step_bf16(const void* z, int64_t ld, const void* in_b, 
     RgArgs a = {z, in_b, o, state, nullptr, conv, conv_b, ra, ra_b, ri, ri_b, decay, pos, nullptr, nullptr, nullptr,
                 ld, (int)W, (int)nb, (int)bs, (int)taps, 1, 0, 1, (int)act, (int)B};
     // more channels per workgroup rebuild the convolution less often, fewer spread the weights over more workgroups
-    static const int cg_env = [] { const char* e = getenv("EVO_RG_CG"); return e ? atoi(e) : 0; }();
-    const int cg = cg_env ? cg_env : (B <= 8 ? 1 : 2);
+    const int cg = B <= 4 ? 1 : (B <= 32 || bs > 256 ? 2 : 4);
     const dim3 grid((unsigned)((bs + 16 * cg - 1) / (16 * cg)), (unsigned)nb, (unsigned)((B + 15) / 16));
 #define RS1(KS, CG) hipLaunchKernelGGL((rglru_step_kernel<KS, CG>), grid, dim3(256 * CG), 0, (hipStream_t)stream, a)
 #define RS(KS) do { if (cg == 1) RS1(KS, 1); else if (cg == 2) RS1(KS, 2); else RS1(KS, 4); } while (0)
-    if (bs <= 64) RS(2); else if (bs <= 96) RS(3); else if (bs <= 128) RS(4); else if (bs <= 192) RS(6); else if (bs <= 256) RS(8); else RS(12);
+    if (bs <= 64) RS(2); else if (bs <= 96) RS(3); else if (bs <= 128) RS(4); else if (bs <= 192) RS(6); else if (bs <= 256) RS(8);
+    else if (cg == 1) RS1(12, 1); else RS1(12, 2);
 #undef RS1
 #undef RS
     return evo_launch_status();

@@ -80,9 +80,9 @@ __global__ __launch_bounds__(64 * NW, MINW) void window_attn_kernel(WinArgs a, i
         for (int db = 0; db < DVB; ++db) o[c][db] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     }
 
-    // eight threads share a row: thread (row rt, dims 8 (tid % 8) + 64 i) of keys rt and (four waves) rt + 32, values of keys 2 rt and 2 rt + 1
-    // (eight waves: rt & 31, half of the dims)
-    const int rt = tid >> 3, ct = (tid & 7) * 8, vt = rt & 31, vi0 = (rt >> 5) * VI;
+    // eight threads share a row: thread (row rt = tid / 8, dims ct + 64 i) of keys rt and (four waves) rt + 32, values of keys 2 vt and 2 vt + 1
+    // (eight waves: half of the value dims each).  A tile's base is uniform, offsets within it are 32 bits; eight waves make them anew for every
+    // tile: held across tiles they spill.
     mx_u32x4 rk[MAPS * KG][KU], rv[VI][2];
     auto any8 = [](const uint16_t* x, int nx, const uint16_t* y, int ny, int d) {       // eight dims of [x (nx) | y (ny) | zeros], any alignment
         uint32_t w[8];
@@ -92,37 +92,44 @@ __global__ __launch_bounds__(64 * NW, MINW) void window_attn_kernel(WinArgs a, i
     };
     // (keys past the end and dimensions past the head's repeat valid ones -- their scores are masked, the queries are zero there, their
     //  outputs are not stored --, so that the aligned form has no branch among its requests)
+    const uint32_t row_bytes = (uint32_t)a.ldkv * 2;
+    auto here = [](int v) __attribute__((always_inline)) {
+        if constexpr (NW == 8) asm volatile("" : "+v"(v));
+        return v;
+    };
     auto load_k = [&](int j0) __attribute__((always_inline)) {
+        const char* tile = (const char*)(kn + j0 * a.ldkv);
+        const int t = here(tid), rt = t >> 3, ct = (t & 7) * 8;
 #pragma unroll
         for (int u = 0; u < KU; ++u) {
-            const int j = j0 + rt + 32 * u < nk ? j0 + rt + 32 * u : nk - 1;
-            const uint16_t *pn = kn + j * a.ldkv, *pr_ = kr + (int64_t)j * a.dr;
+            const int r = rt + 32 * u < nk - j0 ? rt + 32 * u : nk - 1 - j0;
+            const uint16_t *pn = kn + (j0 + r) * a.ldkv, *pr_ = kr + (int64_t)(j0 + r) * a.dr;
 #pragma unroll
             for (int i = 0; i < MAPS * KG; ++i) {
-                const int d = ct + 64 * (i % KG);
-                const uint16_t* pm = pn + (i / KG) * dn;         // (a shared key part goes with one map only)
-                if constexpr (!VEC) rk[i][u] = any8(pm, dn, pr_, a.dr, d);
-                else {
-                    const int dc = d < dh ? d : dh - 8;
-                    rk[i][u] = *(const mx_u32x4*)(MAPS == 2 || dc < dn ? pm + dc : pr_ + (dc - dn));
-                }
+                const int d = ct + 64 * (i % KG), dc = d < dh ? d : dh - 8;
+                if constexpr (!VEC) rk[i][u] = any8(pn + (i / KG) * dn, dn, pr_, a.dr, d);
+                else if constexpr (MAPS == 2)                    // (a shared key part goes with one map only)
+                    rk[i][u] = *(const mx_u32x4*)(tile + ((uint32_t)r * row_bytes + 2u * (uint32_t)((i / KG) * dn + dc)));
+                else rk[i][u] = *(const mx_u32x4*)(dc < dn ? pn + dc : pr_ + (dc - dn));
             }
         }
     };
     auto load_v = [&](int j0) __attribute__((always_inline)) {
+        const char* tile = (const char*)(vg + j0 * a.ldkv);
+        const int t = here(tid), vt = (t >> 3) & 31, vi0 = (t >> 8) * VI, ct = (t & 7) * 8;
 #pragma unroll
         for (int u = 0; u < 2; ++u) {
-            const int j = j0 + 2 * vt + u < nk ? j0 + 2 * vt + u : nk - 1;
-            const uint16_t* pv = vg + j * a.ldkv;
+            const int r = 2 * vt + u < nk - j0 ? 2 * vt + u : nk - 1 - j0;
 #pragma unroll
             for (int i = 0; i < VI; ++i) {
                 const int d = ct + 64 * (vi0 + i);
-                if constexpr (!VEC) rv[i][u] = any8(pv, dv, pv, 0, d);
-                else rv[i][u] = *(const mx_u32x4*)(pv + (d < dv ? d : dv - 8));
+                if constexpr (!VEC) rv[i][u] = any8(vg + (j0 + r) * a.ldkv, dv, vg, 0, d);
+                else rv[i][u] = *(const mx_u32x4*)(tile + ((uint32_t)r * row_bytes + 2u * (uint32_t)(d < dv ? d : dv - 8)));
             }
         }
     };
     auto stage = [&]() __attribute__((always_inline)) {
+        const int t = here(tid), rt = t >> 3, vt = rt & 31, vi0 = (t >> 8) * VI, ct = (t & 7) * 8;
 #pragma unroll
         for (int i = 0; i < MAPS * KG; ++i)
 #pragma unroll
@@ -367,7 +374,7 @@ extern "C" int evo_window_attn(const void* q, int64_t ldq, const void* kn, const
     hipStream_t s = (hipStream_t)stream;
     const int64_t dq = dn + dr;
     if (!f32 && mfma && dq <= (maps == 2 ? 128 : 256) && dv <= 256) {
-        const bool vec = dn % 8 == 0 && dr % 8 == 0 && dv % 8 == 0 && ldq % 8 == 0 && ldkv % 8 == 0 &&
+        const bool vec = dn % 8 == 0 && dr % 8 == 0 && dv % 8 == 0 && ldq % 8 == 0 && ldkv % 8 == 0 && ldkv <= 0xffffff &&
                          (((uintptr_t)q | (uintptr_t)kn | (uintptr_t)v | (uintptr_t)kr) & 15) == 0;
 #define WA1(KS, DVB, QC, VEC, KEEP, MAPS, MINW, NW)                                                                        \
     do {                                                                                                                   \
@@ -379,7 +386,9 @@ extern "C" int evo_window_attn(const void* q, int64_t ldq, const void* kn, const
 #define WAN(KS, DVB, QC, VEC, MAPS, MINW, NW) do { if (kp) WA1(KS, DVB, QC, VEC, true, MAPS, MINW, NW); else WA1(KS, DVB, QC, VEC, false, MAPS, MINW, NW); } while (0)
 #define WA(KS, DVB, QC, VEC, MAPS, MINW) WAN(KS, DVB, QC, VEC, MAPS, MINW, 4)
 #define WAV(KS, QC) do { if (dv <= 64) WA(KS, 4, QC, true, 1, 2); else if (dv <= 128) WA(KS, 8, QC, true, 1, 2); else WA(KS, 16, 1, true, 1, 2); } while (0)
-#define WA2(KS) do { if (dv <= 64) WA(KS, 4, 2, true, 2, 2); else if (dv <= 128) WA(KS, 8, 2, true, 2, 2); else WAN(KS, 16, 2, true, 2, 2, 8); } while (0)
+#define WA2(KS) do { if (dv <= 64) WA(KS, 4, 2, true, 2, 2); else if (dv <= 128) WA(KS, 8, 2, true, 2, 2); \
+                     else if (!kp) WA1(KS, 16, 2, true, false, 2, 2, 8); \
+                     else WA1(KS, 16, 2, true, true, 2, (KS > 2 ? 1 : 2), (KS > 2 ? 4 : 8)); } while (0)   /* (kept tokens cost registers) */
         if (maps == 2) { if (!vec) WA(4, 16, 2, false, 2, 1); else if (dq <= 64) WA2(2); else WA2(4); }
         else if (!vec) { if (dq <= 64 && dv <= 64) WA(2, 4, 2, false, 1, 2); else WA(8, 16, 1, false, 1, 2); }
         else if (dq <= 64) WAV(2, 2);

@@ -98,7 +98,7 @@ def spiky(lq, lk, H, G, maps, n, dv, dt, seed):
 CASES = [(2, 2, 1, 32, 64, 41, 5), (6, 2, 1, 48, 48, 136, 4), (3, 1, 1, 10, 9, 17, 3), (4, 1, 1, 64, 128, 64, 70), (1, 1, 1, 128, 128, 65, 1), (2, 2, 1, 160, 40, 33, 64),
          (2, 1, 1, 192, 128, 63, 2), (1, 1, 1, 256, 256, 100, 9), (8, 2, 1, 16, 24, 1, 1), (2, 2, 1, 300, 300, 33, 7), (2, 2, 1, 24, 200, None, 0), (4, 4, 2, 48, 96, None, 0),
          (4, 2, 2, 64, 64, None, 0), (2, 1, 2, 128, 256, None, 0), (3, 1, 2, 7, 11, None, 0), (2, 2, 2, 96, 128, 50, 6), (1, 1, 2, 16, 160, 64, 0), (2, 2, 2, 150, 20, None, 0),
-         (2, 1, 2, 24, 256, 33, 130), (5, 5, 2, 40, 30, None, 0)]
+         (2, 1, 2, 24, 256, 33, 130), (5, 5, 2, 40, 30, None, 0), (2, 1, 2, 128, 256, 70, 3)]
 
 
 @TYPES

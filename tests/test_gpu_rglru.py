@@ -136,7 +136,7 @@ def test_slow_decays_carry_far(ops):
 
 @TYPES
 @pytest.mark.parametrize("W,nb,taps", SIZES)
-@pytest.mark.parametrize("B", [1, 5, 16, 19])
+@pytest.mark.parametrize("B", [1, 5, 16, 19, 40])
 def test_recurrence_step(ops, dt, W, nb, taps, B):
     """Tokens one by one from a sequence's start: bias and activation in the kernel, rows at different positions, other rows untouched."""
     from evo_amd.mixer_ops import TokenBatch

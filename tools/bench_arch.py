@@ -3,6 +3,7 @@ models of the same width, depth and feed-forward weights, through prompt passes 
 the part's peak each reaches.  Run as `python bench.py --arch vozalorn` or `--arch batodra`."""
 import json
 import math
+import sys
 import time
 
 import torch
@@ -55,6 +56,10 @@ def build(kind, n_layers, device):
     if kind == "stripedhyena":
         m.prepare()
     return m
+
+
+def progress(line):
+    print(line, file=sys.stderr, flush=True)
 
 
 def weight_bytes(m):
@@ -151,6 +156,7 @@ class Alone:
 
     def put(self, name, fn, nbytes=0, flop=0, n=20):
         us = captured(fn, n)
+        progress(f"{name}: {us:.1f} us")
         self.out[name] = [round(us, 1), round(max(nbytes / HBM, flop / MFMA) / (us * 1e-6), 3)]
 
     def pairs(self, B, T, heads, window=None, keep=0):
@@ -292,6 +298,7 @@ def run(device, arch="vozalorn", n_layers=8, steps=10):
                 s = seconds(lambda: m.hidden_states(ids), steps)
                 r[f"prefill_{B}x{T}"] = {"tokens_per_s": round(B * T / s), "ms": round(s * 1e3, 3),
                                          "kernels": with_fractions(kernel_times(m, lambda: m.hidden_states(ids)), prefill_work(B, T))}
+                progress(f"{kind} prefill {B} x {T}: {s * 1e3:.2f} ms")
             for B, ctx in ((1, 2048), (8, 2048), (32, 2048)):
                 pool = DecodePool(m, CharLevelTokenizer(512), n_slots=B, device=device)
                 first = pool.prefill([torch.randint(0, 512, (ctx,), device=device)])[0]
@@ -300,6 +307,7 @@ def run(device, arch="vozalorn", n_layers=8, steps=10):
                 r[f"decode_{B}x{ctx}"] = {"tokens_per_s": round(B / s), "us_per_step": round(s * 1e6, 1),
                                           "weights_of_hbm_peak": round(weight_bytes(m) / s / HBM, 3), "captured": pool._graph is not None,
                                           "kernels": with_fractions(kernel_times(m, pool._step_eager), decode_work(B, ctx))}
+                progress(f"{kind} decode {B} x {ctx}: {s * 1e6:.0f} us")
                 del pool
         del m
         torch.cuda.empty_cache()
