@@ -95,8 +95,8 @@ def spiky(lq, lk, H, G, maps, n, dv, dt, seed):
     return [t.to(dt) for t in (q, k, v)]
 
 
-CASES = [(2, 2, 1, 32, 64, 41, 5), (6, 2, 1, 48, 48, 136, 4), (3, 1, 1, 10, 9, 17, 3), (4, 1, 1, 64, 128, 64, 70), (1, 1, 1, 128, 128, 65, 1), (2, 2, 1, 160, 40, 33, 64),
-         (2, 1, 1, 192, 128, 63, 2), (1, 1, 1, 256, 256, 100, 9), (8, 2, 1, 16, 24, 1, 1), (2, 2, 1, 300, 300, 33, 7), (2, 2, 1, 24, 200, None, 0), (4, 4, 2, 48, 96, None, 0),
+CASES = [(2, 2, 1, 32, 64, 41, 5), (6, 2, 1, 56, 40, 120, 6), (3, 1, 1, 10, 9, 17, 3), (4, 1, 1, 64, 128, 64, 70), (1, 1, 1, 128, 128, 65, 1), (2, 2, 1, 160, 40, 33, 64),
+         (2, 1, 1, 192, 128, 63, 2), (1, 1, 1, 256, 256, 100, 9), (8, 2, 1, 16, 24, 1, 1), (2, 2, 1, 300, 300, 33, 7), (2, 2, 1, 24, 200, None, 0), (3, 3, 2, 56, 112, None, 0),
          (4, 2, 2, 64, 64, None, 0), (2, 1, 2, 128, 256, None, 0), (3, 1, 2, 7, 11, None, 0), (2, 2, 2, 96, 128, 50, 6), (1, 1, 2, 16, 160, 64, 0), (2, 2, 2, 150, 20, None, 0),
          (2, 1, 2, 24, 256, 33, 130), (5, 5, 2, 40, 30, None, 0), (2, 1, 2, 128, 256, 70, 3)]
 
@@ -134,8 +134,8 @@ def test_query_that_sees_one_token_only(ops, mfma):
 # ------------------------------------------------------------------------------------------------ decode
 @TYPES
 @pytest.mark.parametrize("H,G,maps,n,dv,keep,window", [
-    (2, 2, 1, 32, 64, 3, 9), (6, 2, 1, 48, 48, 4, 136), (3, 1, 1, 10, 9, 1, 20), (40, 2, 1, 64, 128, 0, 64), (4, 4, 1, 128, 128, 2, 300), (2, 1, 1, 256, 256, 0, 33),
-    (2, 2, 1, 300, 300, 5, 40), (4, 1, 1, 96, 200, 0, 1), (4, 4, 2, 48, 96, 0, 700), (17, 1, 2, 64, 64, 0, 200), (2, 1, 2, 128, 256, 0, 130), (3, 1, 2, 7, 11, 0, 50),
+    (2, 2, 1, 32, 64, 3, 9), (6, 2, 1, 56, 40, 6, 120), (3, 1, 1, 10, 9, 1, 20), (40, 2, 1, 64, 128, 0, 64), (4, 4, 1, 128, 128, 2, 300), (2, 1, 1, 256, 256, 0, 33),
+    (2, 2, 1, 300, 300, 5, 40), (4, 1, 1, 96, 200, 0, 1), (3, 3, 2, 56, 112, 0, 700), (17, 1, 2, 64, 64, 0, 200), (2, 1, 2, 128, 256, 0, 130), (3, 1, 2, 7, 11, 0, 50),
     (2, 2, 2, 24, 40, 7, 65), (2, 2, 2, 150, 20, 0, 70)])
 def test_decode_attention(ops, mfma, dt, H, G, maps, n, dv, keep, window):
     if not mfma and dt == F32:
